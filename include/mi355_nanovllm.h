@@ -736,11 +736,17 @@ int mi_moe_combine_f32(const float* y, const float* h, int64_t ldh, const int32_
 #define MI_ACT_SOFTCAP   5  /* alpha tanh(z / alpha): the epilogue's alpha is the cap (mi_gemm_any_act, no w2) */
 #define MI_ACT_CLAMPED_GLU 6 /* two weights: g = min(x w^T, limit), u = clamp(x w2^T, -limit, limit);
                               * y = g sigmoid(1.702 g) (u + 1)  (mi_gemm_any_grouped_glu) */
+#define MI_ACT_TANH      7
+#define MI_ACT_DECAY     8  /* exp(-exp(-1/2) sigmoid(z)): a decay between exp(-exp(-1/2)) and 1 */
 /* mi_gemm_any with an epilogue: v = x w^T + bias (bias may be NULL); w2 != NULL: y = alpha * act(v) * (x w2^T + bias2),
  * else y = alpha * act(v). */
 int mi_gemm_any_act(const float* x, int64_t ldx, const void* w, const void* w2, int w_dtype, const float* bias,
                     const float* bias2, int act, float* y, int64_t ldy, int M, int N, int K, float alpha, int exact,
                     mi_stream stream);
+/* y = x w^T + bias with an activation per range of features: none below act_from, `act` from act_from on, `act2` from
+ * act2_from (>= act_from) on - projections of one input that need different activations as one product. */
+int mi_gemm_any_segments(const float* x, int64_t ldx, const void* w, int w_dtype, const float* bias, int act, int act_from,
+                         int act2, int act2_from, float* y, int64_t ldy, int M, int N, int K, int exact, mi_stream stream);
 /* mi_gemm_any_grouped with the activation named: y = act(x w^T) (* (x w2^T) with w2). */
 int mi_gemm_any_grouped_act(const float* x, int64_t ldx, const int32_t* x_rows, const void* w, const void* w2, int w_dtype,
                             int act, const int32_t* group_offsets, int n_groups, int rows_per_group_max, float* y,
@@ -778,11 +784,13 @@ int mi_paged_attention_f32(const float* q, int64_t ldq, const void* k_cache, con
  * softcap * tanh(s / softcap) before the mask and the softmax.  value_heads (a divisor of G): the value cache has this many
  * heads, [blocks][value_heads][block_size][.], query head h reads value head h / (H / value_heads) - with fewer, wider value
  * heads than key heads (a token's value heads side by side in one row, v_cache possibly pointing at a column of it) every
- * query head weighs the values of several key/value heads at once: out [rows][H][Dv] with Dv the width read. */
+ * query head weighs the values of several key/value heads at once: out [rows][H][Dv] with Dv the width read.  The same
+ * with narrow value heads lets several key heads SHARE a value head (maps of one head over the same values).
+ * chunk > 0: position i sees only the keys of its own chunk, floor(i / chunk) = floor(j / chunk), on top of the window. */
 int mi_paged_attention_ext(const float* q, int64_t ldq, const void* k_cache, const void* v_cache, int64_t ldv,
                            int cache_dtype, const int32_t* block_tables, int table_cols, const int32_t* cu_q,
                            const int32_t* kv_lens, int n_seqs, int rows, int H, int G, int D, int Dv, int block_size,
-                           int window, float scale, int bias_kind, const float* bias_p1, const float* bias_p2,
+                           int window, int chunk, float scale, int bias_kind, const float* bias_p1, const float* bias_p2,
                            const float* sink, float softcap, int value_heads, const float* gate, int64_t ldg, float* out,
                            int64_t ldo, float* workspace, int64_t workspace_elems, mi_stream stream);
 /* res += mult * y (y may be NULL); w != NULL: out = res / sqrt(mean(res^2) + eps) * (w + shift) per row. */
@@ -869,10 +877,42 @@ int mi_rotary_store(float* proj, int64_t ld, int q_off, int k_off, int v_off, in
  * in the chunk (the others are left alone). */
 int mi_head_mix(const float* o, int64_t ldo_in, const float* talk, int rows, int H, int G, int Dv, int c0, int n_chunk,
                 float out_scale, float* out, int64_t ldo, mi_stream stream);
-/* out[row][h] <- out_scale * out / sqrt(mean over Dv + eps) (* norm_w [Dv] if not NULL) (* act(gate_pre[row][h]) if not
+/* out[row][h] <- out_scale * out / sqrt(mean over Dv + eps) (* norm_w if not NULL: [Dv] for every head with norm_stride 0,
+ * [H][Dv] with norm_stride Dv) (* act(gate_pre[row][h]) if not
  * NULL, gate_act = MI_ACT_SIGMOID or MI_ACT_SILU), in place: the per-head norm and gate of a recurrence's read-out. */
 int mi_head_norm_gate(float* out, int64_t ldo, const float* gate_pre, int64_t ld_gate, int gate_act, const float* norm_w,
-                      float out_scale, int rows, int H, int Dv, float eps, mi_stream stream);
+                      int norm_stride, float out_scale, int rows, int H, int Dv, float eps, mi_stream stream);
+
+/* Residual STREAMS: n_streams copies of the residual per row, [rows][n_streams][width] (ld_* = floats between rows, *_stride
+ * between a row's streams; src_stride 0: every stream is the same row - the embedding).  One launch is a sublayer boundary:
+ *   y != NULL    dst_t = sum_s mix[s][t] src_s + out_coef[t] y   (all t from the old streams)         else the streams are src's
+ *   u = sum_s in_coef[s] stream_s                                (in_coef == NULL: ones)
+ *   norm_w       h = u cut into `groups` equal parts, each / sqrt(mean(part^2) + eps), the whole * norm_w   (NULL: h = u)
+ *   shift        h_t <- h_t + (h_{t-1} - h_t) * shift per channel, h_{t-1} being the previous position's h before its own
+ *                shift: the row before, the slot's shift_state [slots][width] (what the sequence's last row of the step before
+ *                left there) or zeros at position 0; the state is advanced.  Steps with several rows of a sequence
+ *                (max_rows_per_seq > 1) need carry [n_seqs][width] and dst != src.
+ * dst == NULL: the new streams are not stored (the last boundary).  cu_q, kv_lens, slot_ids: as in mi_causal_conv; needed
+ * with shift only.  n_streams <= 8, width <= 8000. */
+int mi_stream_mix(const float* src, int64_t ld_src, int64_t src_stride, float* dst, int64_t ld_dst, int64_t dst_stride,
+                  int n_streams, const float* y, int64_t ldy, const float* mix, const float* out_coef, const float* in_coef,
+                  const float* norm_w, int groups, float eps, const float* shift, float* shift_state, float* carry,
+                  const int32_t* cu_q, const int32_t* kv_lens, const int32_t* slot_ids, int n_seqs, int max_rows_per_seq,
+                  float* h, int64_t ldh, int rows, int width, mi_stream stream);
+/* Differential heads: o [rows][G][2][H / G][Dv] holds, per key/value head, the read-outs of map 1 and of map 2 of its query
+ * heads; lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff with lam [4][D] = lq1, lk1, lq2, lk2;
+ * out[row][h] = (a1 - lambda a2) / sqrt(mean over Dv + eps) * (1 - diff) (* sigmoid(gate[row][h]) if not NULL: a number per
+ * head). */
+int mi_diff_heads(const float* o, int64_t ldo_in, const float* lam, int D, float diff, float eps, const float* gate,
+                  int64_t ldg, float* out, int64_t ldo, int rows, int H, int G, int Dv, mi_stream stream);
+/* Generalised delta rule, fp32 state [slots][mi_general_delta_state_elems] (thread-order layout; -1: D > 256).  Per head,
+ * u = k / sqrt(sum k^2 + 1e-6):  S <- diag(w) S - (a u) (u^T S) + k v^T (both terms from the old S);  o = S^T r.
+ * proj rows hold r, k, a [H*D] and v [H*Dv] at the given columns (a: the removal rate as it is used), w_decay [rows][H*D] the
+ * decay per head and key channel.  out [rows][H*Dv]: the raw read-out. */
+int64_t mi_general_delta_state_elems(int H, int D, int Dv);
+int mi_general_delta(const float* proj, int64_t ld, int r_off, int k_off, int v_off, int a_off, const float* w_decay,
+                     int64_t ldw, float* state, const int32_t* cu_q, const int32_t* kv_lens, const int32_t* slot_ids,
+                     int n_seqs, int rows, int H, int D, int Dv, float* out, int64_t ldo, mi_stream stream);
 
 /* ---- host-side hashing (reference: engine/block_manager.py:38-44) --------- */
 /* xxh64 of `len` bytes with seed 0, optionally prefixed by the 8 little-endian

@@ -51,6 +51,10 @@ struct GemmAnyArgs {
   const float* row_scale;
   const int32_t* row_scale_rows;
   float limit;  // MI_ACT_CLAMPED_GLU
+  // act_segments: `act` applies to the features n >= act_from only, `act2` to those from act2_from (>= act_from) on -
+  // several projections of one input, each with an activation of its own, as one product
+  bool act_segments;
+  int act_from, act2, act2_from;
 };
 
 template <typename TW>
@@ -68,6 +72,8 @@ __device__ __forceinline__ float act_f(int act, float z) {
     case MI_ACT_GELU_TANH: return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
     case MI_ACT_GELU_ERF: return 0.5f * z * (1.f + erff(z * 0.7071067811865476f));
     case MI_ACT_SIGMOID: return 1.f / (1.f + expf(-z));
+    case MI_ACT_TANH: return tanhf(z);
+    case MI_ACT_DECAY: return expf(-0.6065306597126334f / (1.f + expf(-z)));  // exp(-exp(-1/2) sigmoid(z))
     default: return z;  // (MI_ACT_SOFTCAP is finish()'s: it needs the cap)
   }
 }
@@ -87,6 +93,8 @@ __device__ __forceinline__ float finish(const GemmAnyArgs& a, int64_t m, int64_t
     } else {
       v = act_f(a.act, v) * v2;
     }
+  } else if (a.act_segments) {
+    if (n >= a.act_from) v = n >= a.act2_from ? act_f(a.act2, v) : act_f(a.act, v);
   } else {
     v = a.act == MI_ACT_SOFTCAP ? tanhf(v / a.alpha) : act_f(a.act, v);  // (times alpha below: alpha tanh(v / alpha))
   }
@@ -541,7 +549,9 @@ static int gemm_any_dispatch(const GemmAnyArgs& a, int w_dtype, int groups, int 
   return MI_EINVAL;
 }
 
-static bool act_ok(int act) { return act >= MI_ACT_NONE && act <= MI_ACT_SOFTCAP; }
+static bool act_ok(int act) {
+  return (act >= MI_ACT_NONE && act <= MI_ACT_SOFTCAP) || act == MI_ACT_TANH || act == MI_ACT_DECAY;
+}
 
 extern "C" int mi_gemm_any(const float* x, int64_t ldx, const void* w, int w_dtype, float* y, int64_t ldy, int M, int N,
                            int K, float alpha, int exact, mi_stream stream) {
@@ -553,7 +563,16 @@ extern "C" int mi_gemm_any_act(const float* x, int64_t ldx, const void* w, const
                                int exact, mi_stream stream) {
   if (!x || !w || !y || M < 0 || N < 0 || K < 1 || ldx < K || ldy < N || !act_ok(act) || (bias2 && !w2)) return MI_EINVAL;
   if (act == MI_ACT_SOFTCAP && (w2 || !(alpha > 0.f))) return MI_EINVAL;
-  GemmAnyArgs a{x, ldx, w, w2, y, ldy, M, N, K, alpha, nullptr, nullptr, nullptr, bias, bias2, act, nullptr, 0, 0, 0, 0, nullptr, nullptr, 0.f};
+  GemmAnyArgs a{x, ldx, w, w2, y, ldy, M, N, K, alpha, nullptr, nullptr, nullptr, bias, bias2, act, nullptr, 0, 0, 0, 0, nullptr, nullptr, 0.f, false, 0, 0, 0};
+  return gemm_any_dispatch(a, w_dtype, 1, M, exact ? 1 : 0, S(stream));
+}
+
+extern "C" int mi_gemm_any_segments(const float* x, int64_t ldx, const void* w, int w_dtype, const float* bias, int act,
+                                    int act_from, int act2, int act2_from, float* y, int64_t ldy, int M, int N, int K,
+                                    int exact, mi_stream stream) {
+  if (!x || !w || !y || M < 0 || N < 0 || K < 1 || ldx < K || ldy < N || !act_ok(act) || !act_ok(act2)) return MI_EINVAL;
+  if (act == MI_ACT_SOFTCAP || act2 == MI_ACT_SOFTCAP || act_from < 0 || act2_from < act_from) return MI_EINVAL;
+  GemmAnyArgs a{x, ldx, w, nullptr, y, ldy, M, N, K, 1.0f, nullptr, nullptr, nullptr, bias, nullptr, act, nullptr, 0, 0, 0, 0, nullptr, nullptr, 0.f, true, act_from, act2, act2_from};
   return gemm_any_dispatch(a, w_dtype, 1, M, exact ? 1 : 0, S(stream));
 }
 
@@ -563,7 +582,7 @@ extern "C" int mi_gemm_any_batched(const float* x, int64_t ldx, int64_t x_batch,
   if (!x || !w || !y || n_batch < 1 || M < 0 || N < 0 || K < 1 || ldx < K || ldy < N) return MI_EINVAL;
   if (n_batch > 65535) return MI_EUNSUPPORTED;
   GemmAnyArgs a{x, ldx, w, nullptr, y, ldy, M, N, K, 1.0f, nullptr, nullptr, nullptr, nullptr, nullptr, MI_ACT_NONE,
-                gate, ldgate, x_batch, y_batch, gate_batch, nullptr, nullptr, 0.f};
+                gate, ldgate, x_batch, y_batch, gate_batch, nullptr, nullptr, 0.f, false, 0, 0, 0};
   return gemm_any_dispatch(a, w_dtype, n_batch, M, exact ? 1 : 0, S(stream));
 }
 
@@ -596,6 +615,6 @@ extern "C" int mi_gemm_any_grouped_glu(const float* x, int64_t ldx, const int32_
   if (row_scale_rows && !row_scale) return MI_EINVAL;
   if (n_groups > 65535) return MI_EUNSUPPORTED;
   GemmAnyArgs a{x, ldx, w, w2, y, ldy, rows_per_group_max, N, K, 1.0f, group_offsets, x_rows, y_rows, nullptr, nullptr,
-                act, nullptr, 0, 0, 0, 0, row_scale, row_scale_rows, limit};
+                act, nullptr, 0, 0, 0, 0, row_scale, row_scale_rows, limit, false, 0, 0, 0};
   return gemm_any_dispatch(a, w_dtype, n_groups, rows_per_group_max, exact ? 1 : 0, S(stream));
 }

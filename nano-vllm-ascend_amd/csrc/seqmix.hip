@@ -33,41 +33,9 @@
 // of prompt portions, whose two products take q and the softmax weights as bf16 hi + lo pairs: fp32 quantities to 2^-17).
 // A step's rows are described by cu_q [n_seqs + 1] (row range of each sequence) and kv_lens [n_seqs] (the sequence's
 // length INCLUDING this step's rows): row r of sequence s sits at position kv_lens[s] - (cu_q[s+1] - cu_q[s]) + r.
-#include "mi_common.hpp"
+#include "seqmix_common.hpp"
 
 namespace mi {
-
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.f / (1.f + expf(-z)); }
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
-
-template <typename T>
-__device__ __forceinline__ float ld_f(const T* p);
-template <>
-__device__ __forceinline__ float ld_f<float>(const float* p) { return *p; }
-template <>
-__device__ __forceinline__ float ld_f<uint16_t>(const uint16_t* p) { return bf2f(*p); }
-template <typename T>
-__device__ __forceinline__ void st_f(T* p, float v);
-template <>
-__device__ __forceinline__ void st_f<float>(float* p, float v) { *p = v; }
-template <>
-__device__ __forceinline__ void st_f<uint16_t>(uint16_t* p, float v) { *p = f2bf(v); }
-
-// sum over a 256-thread workgroup; every thread gets the result.  red: 4 floats of LDS per concurrent reduction.
-__device__ __forceinline__ float block_sum256(float v, float* red) {
-  v = wave_sum(v);
-  __syncthreads();  // (red may still be read from the previous reduction)
-  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
-  __syncthreads();
-  return (red[0] + red[1]) + (red[2] + red[3]);
-}
-
-// the sequence a step row belongs to (n_seqs is small: a linear walk, identical on every lane)
-__device__ __forceinline__ int seq_of_row(const int32_t* cu_q, int n_seqs, int row) {
-  int s = 0;
-  while (s + 1 < n_seqs && row >= cu_q[s + 1]) ++s;
-  return s;
-}
 
 template <typename TT>
 __global__ __launch_bounds__(256) void embedding_f32_kernel(const int64_t* __restrict__ ids, const TT* __restrict__ table,
@@ -155,6 +123,8 @@ __global__ __launch_bounds__(256) void swa_prepare_kernel(float* __restrict__ pr
 // h / (H / value_heads)) - fewer, wider value heads than key heads let every query head weigh the values of SEVERAL
 // key/value heads at once (value rows holding the heads side by side), which is what mixing the heads' softmax weights
 // afterwards needs.
+// chunk > 0: position i sees the keys of its own chunk only (floor(i / chunk) = floor(j / chunk), positions counted from
+// the sequence's start); with the window: both hold.
 struct AttnBias {
   int kind;
   const float* p1;
@@ -162,7 +132,14 @@ struct AttnBias {
   const float* sink;
   float softcap;
   int value_heads;
+  int chunk;
 };
+// the oldest key position `pos` sees
+__device__ __forceinline__ int first_key(const AttnBias& bias, int pos, int window) {
+  int lo = max(0, pos - window + 1);
+  if (bias.chunk > 0) lo = max(lo, pos - pos % bias.chunk);
+  return lo;
+}
 __device__ __forceinline__ float capped(const AttnBias& bias, float s) {
   return bias.softcap > 0.f ? bias.softcap * tanhf(s / bias.softcap) : s;
 }
@@ -218,7 +195,7 @@ __global__ __launch_bounds__(256) void swa_attention_kernel(const float* __restr
   for (int d = lane; d < D; d += 64) qs[d] = q[(int64_t)row * ldq + h * D + d];
   const int s = seq_of_row(cu_q, n_seqs, row);
   const int pos = kv_lens[s] - (cu_q[s + 1] - cu_q[s]) + (row - cu_q[s]);
-  const int lo = max(0, pos - window + 1);
+  const int lo = first_key(bias, pos, window);
   const int g = h / (H / G);
   const int Gv = bias.value_heads, gv = h / (H / Gv);
   const HeadBias hb = head_bias(bias, h, H);
@@ -332,7 +309,10 @@ __global__ __launch_bounds__(256) void swa_attention_vec_kernel(const float* __r
     for (int r = 0; r < nr; ++r)
       for (int d = lane; d < D; d += 64) qs[r * D + d] = q[(int64_t)(first + r) * ldq + h * D + d];
     __builtin_amdgcn_wave_barrier();
-    const int lo = max(0, pos0 - window + 1), hi = pos0 + nr - 1;
+    const int lo = first_key(bias, pos0, window), hi = pos0 + nr - 1;
+    int row_lo[RPW];
+#pragma unroll
+    for (int r = 0; r < RPW; ++r) row_lo[r] = first_key(bias, pos0 + r, window);
     float m[RPW], l[RPW], acc[RPW][VEC];
 #pragma unroll
     for (int r = 0; r < RPW; ++r) {
@@ -366,7 +346,7 @@ __global__ __launch_bounds__(256) void swa_attention_vec_kernel(const float* __r
 #pragma unroll
       for (int r = 0; r < RPW; ++r) {
         const int pos = pos0 + r;
-        const bool vis = r < nr && j <= pos && j > pos - window;
+        const bool vis = r < nr && j <= pos && j >= row_lo[r];
         const float sc = vis ? capped(bias, dots[r] * scale - dist_bias(hb, pos - j)) : -INFINITY;
         const float m_new = fmaxf(m[r], wave_max(sc));
         const float p = vis ? expf(sc - m_new) : 0.f;
@@ -500,8 +480,9 @@ __global__ __launch_bounds__(256) void swa_attention_mfma_kernel(const float* __
       qh[ks] = as_frag(u32x4{pack_bf(xv[0], xv[1]), pack_bf(xv[2], xv[3]), pack_bf(xv[4], xv[5]), pack_bf(xv[6], xv[7])});
       ql[ks] = as_frag(u32x4{pack_bf(lo[0], lo[1]), pack_bf(lo[2], lo[3]), pack_bf(lo[4], lo[5]), pack_bf(lo[6], lo[7])});
     }
-    const int lo_key = max(0, pos0 - window + 1), hi_key = pos0 + nr - 1;
+    const int lo_key = first_key(bias, pos0, window), hi_key = pos0 + nr - 1;
     const int my_pos = pos0 + qi;
+    const int my_lo = first_key(bias, my_pos, window);
     float m = -INFINITY, l = 0.f;
     f32x4 oacc[DVM];
 #pragma unroll
@@ -531,7 +512,7 @@ __global__ __launch_bounds__(256) void swa_attention_mfma_kernel(const float* __
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         const int key = j0 + (e >> 2) * 16 + kg * 4 + (e & 3);
-        vis[e] = qi < nr && key <= my_pos && key > my_pos - window;
+        vis[e] = qi < nr && key <= my_pos && key >= my_lo;
         sc[e] = sacc[e >> 2][e & 3] * scale;
         dist[e] = my_pos - key;
       }
@@ -683,7 +664,7 @@ __global__ __launch_bounds__(256) void paged_attention_heads_mfma_kernel(
     qh[ks] = as_frag(u32x4{pack_bf(xv[0], xv[1]), pack_bf(xv[2], xv[3]), pack_bf(xv[4], xv[5]), pack_bf(xv[6], xv[7])});
     ql[ks] = as_frag(u32x4{pack_bf(lo[0], lo[1]), pack_bf(lo[2], lo[3]), pack_bf(lo[4], lo[5]), pack_bf(lo[6], lo[7])});
   }
-  const int lo_key = max(0, pos - window + 1), hi_key = pos;
+  const int lo_key = first_key(bias, pos, window), hi_key = pos;
   float m = -INFINITY, l = 0.f;
   f32x4 oacc[DVM];
 #pragma unroll
@@ -1150,11 +1131,12 @@ __global__ __launch_bounds__(kDeltaThreads) void channel_delta_kernel(const floa
 }
 
 // out[row][h] <- out_scale * out / rms(out over Dv) * norm_w (* act(gate) with a gate; norm_w may be nullptr: no weight;
-// gate_act: MI_ACT_SIGMOID or MI_ACT_SILU): one wave per (row, head), in place
+// norm_stride: 0 - one weight [Dv] for every head - or Dv - a weight of its own per head; gate_act: MI_ACT_SIGMOID or
+// MI_ACT_SILU): one wave per (row, head), in place
 __global__ __launch_bounds__(256) void delta_finish_kernel(float* __restrict__ out, int64_t ldo,
                                                            const float* __restrict__ gate_pre, int64_t ld_gate,
-                                                           const float* __restrict__ norm_w, int n_rows, int H, int Dv,
-                                                           float eps, int gate_act, float out_scale) {
+                                                           const float* __restrict__ norm_w, int norm_stride, int n_rows,
+                                                           int H, int Dv, float eps, int gate_act, float out_scale) {
   const int lane = threadIdx.x & 63;
   const int wid = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (wid >= n_rows * H) return;
@@ -1165,7 +1147,7 @@ __global__ __launch_bounds__(256) void delta_finish_kernel(float* __restrict__ o
   const float rstd = out_scale / sqrtf(wave_sum(sq) / (float)Dv + eps);
   for (int d = lane; d < Dv; d += 64) {
     float v = o[d] * rstd;
-    if (norm_w) v *= norm_w[d];
+    if (norm_w) v *= norm_w[h * norm_stride + d];
     if (gate_pre) {
       const float z = gate_pre[(int64_t)row * ld_gate + h * Dv + d];
       v *= gate_act == MI_ACT_SILU ? z * sigmoid_f(z) : sigmoid_f(z);
@@ -2071,25 +2053,26 @@ extern "C" int mi_paged_attention_f32(const float* q, int64_t ldq, const void* k
                                       float* out, int64_t ldo, float* workspace, int64_t workspace_elems,
                                       mi_stream stream) {
   return mi_paged_attention_ext(q, ldq, k_cache, v_cache, ldv, cache_dtype, block_tables, table_cols, cu_q, kv_lens, n_seqs,
-                                rows, H, G, D, Dv, block_size, window, scale, bias_kind, bias_p1, bias_p2, sink, 0.f, G,
+                                rows, H, G, D, Dv, block_size, window, 0, scale, bias_kind, bias_p1, bias_p2, sink, 0.f, G,
                                 gate, ldg, out, ldo, workspace, workspace_elems, stream);
 }
 
 extern "C" int mi_paged_attention_ext(const float* q, int64_t ldq, const void* k_cache, const void* v_cache, int64_t ldv,
                                       int cache_dtype, const int32_t* block_tables, int table_cols, const int32_t* cu_q,
                                       const int32_t* kv_lens, int n_seqs, int rows, int H, int G, int D, int Dv,
-                                      int block_size, int window, float scale, int bias_kind, const float* bias_p1,
-                                      const float* bias_p2, const float* sink, float softcap, int value_heads,
+                                      int block_size, int window, int chunk, float scale, int bias_kind,
+                                      const float* bias_p1, const float* bias_p2, const float* sink, float softcap,
+                                      int value_heads,
                                       const float* gate, int64_t ldg, float* out, int64_t ldo, float* workspace,
                                       int64_t workspace_elems, mi_stream stream) {
   if (!q || !k_cache || !v_cache || !block_tables || !cu_q || !kv_lens || !out || rows < 0 || n_seqs < 1) return MI_EINVAL;
   if (H < 1 || G < 1 || H % G || D < 1 || Dv < 1 || block_size < 1 || window < 1 || table_cols < 1 || ldv < Dv) return MI_EINVAL;
-  if (value_heads < 1 || G % value_heads || !(softcap >= 0.f)) return MI_EINVAL;
+  if (value_heads < 1 || G % value_heads || !(softcap >= 0.f) || chunk < 0) return MI_EINVAL;
   if (bias_kind != MI_BIAS_SLOPE && bias_kind != MI_BIAS_LOG && bias_kind != MI_BIAS_NONE) return MI_EINVAL;
   if (bias_kind == MI_BIAS_LOG && (!bias_p1 || !bias_p2)) return MI_EINVAL;
   if (Dv > 512 || D > 4096) return MI_EUNSUPPORTED;
   if (rows == 0) return MI_OK;
-  const AttnBias bias{bias_kind, bias_p1, bias_p2, sink, softcap, value_heads};
+  const AttnBias bias{bias_kind, bias_p1, bias_p2, sink, softcap, value_heads, chunk};
   if (cache_dtype == MI_DTYPE_BF16)
     return launch_swa<uint16_t>(q, ldq, k_cache, v_cache, block_tables, table_cols, cu_q, kv_lens, n_seqs, rows, H, G, D,
                                 Dv, block_size, window, scale, bias, ldv, gate, ldg, out, ldo, workspace, workspace_elems,
@@ -2186,7 +2169,7 @@ extern "C" int mi_channel_delta(const float* qkv, int64_t ld, int q_off, int k_o
 #undef MI_DELTA
   if (check_launch() != MI_OK) return MI_ELAUNCH;
   hipLaunchKernelGGL(delta_finish_kernel, dim3((n_rows * H + 3) / 4), dim3(256), 0, S(stream), out, ldo, gate_pre,
-                     ld_gate, norm_w, n_rows, H, Dv, eps, MI_ACT_SIGMOID, 1.f);
+                     ld_gate, norm_w, 0, n_rows, H, Dv, eps, MI_ACT_SIGMOID, 1.f);
   return check_launch();
 }
 
@@ -2392,7 +2375,7 @@ extern "C" int mi_linear_attention(const float* proj, int64_t ld, int q_off, int
                        H * Dv, eps);
   else
     hipLaunchKernelGGL(delta_finish_kernel, dim3((n_rows * H + 3) / 4), dim3(256), 0, S(stream), out, ldo, gate_pre,
-                       ld_gate, norm_w, n_rows, H, Dv, eps, MI_ACT_SIGMOID, 1.f);
+                       ld_gate, norm_w, 0, n_rows, H, Dv, eps, MI_ACT_SIGMOID, 1.f);
   return check_launch();
 }
 
@@ -2436,12 +2419,12 @@ extern "C" int mi_head_mix(const float* o, int64_t ldo_in, const float* talk, in
 }
 
 extern "C" int mi_head_norm_gate(float* out, int64_t ldo, const float* gate_pre, int64_t ld_gate, int gate_act,
-                                 const float* norm_w, float out_scale, int rows, int H, int Dv, float eps,
-                                 mi_stream stream) {
+                                 const float* norm_w, int norm_stride, float out_scale, int rows, int H, int Dv,
+                                 float eps, mi_stream stream) {
   if (!out || rows < 0 || H < 1 || Dv < 1 || ldo < (int64_t)H * Dv || (gate_pre && ld_gate < (int64_t)H * Dv)) return MI_EINVAL;
-  if (gate_act != MI_ACT_SIGMOID && gate_act != MI_ACT_SILU) return MI_EINVAL;
+  if ((gate_act != MI_ACT_SIGMOID && gate_act != MI_ACT_SILU) || (norm_stride != 0 && norm_stride != Dv)) return MI_EINVAL;
   if (rows == 0) return MI_OK;
   hipLaunchKernelGGL(delta_finish_kernel, dim3((rows * H + 3) / 4), dim3(256), 0, S(stream), out, ldo, gate_pre, ld_gate,
-                     norm_w, rows, H, Dv, eps, gate_act, out_scale);
+                     norm_w, norm_stride, rows, H, Dv, eps, gate_act, out_scale);
   return check_launch();
 }

@@ -30,6 +30,9 @@ class RowSteps:
             free, total = torch.cuda.mem_get_info(self.device)
             budget = total * cfg.gpu_memory_utilization - (total - free) - n_slots * self.model.state_bytes_per_slot()
             cfg.num_kvcache_blocks = int(budget) // per_block
+            if self.model.cache_bytes_per_block(self.block_size, item) == 0:
+                # (recurrent layers only: pages cost nothing - as many as the longest sequences can ask for)
+                cfg.num_kvcache_blocks = cfg.max_num_seqs * -(-cfg.max_model_len // self.block_size) + 1
         assert cfg.num_kvcache_blocks > 1, "no memory left for the K/V pages"
         self.n_state_slots = n_slots
         # (one slot more than the scheduler hands out: the padded rows of a captured step write their state there)

@@ -38,6 +38,13 @@ configuration:
                             projection, one merged output projection of the two scaled read-outs
   InputWeightedSparseMLP    top-k experts by sigmoid score whose weight multiplies the expert's INPUT; experts
                             W_d (g sigmoid(1.702 g) (u + 1)) with g capped and u clamped
+  StreamResidual            several copies ("streams") of the residual per token: a sublayer reads a weighted sum of them
+                            (normed in groups of channels, optionally shifted towards the previous token's) and its output
+                            goes back into all of them, mixed among themselves
+  TokenShift                h <- h + (h of the previous token - h) * shift per channel; that h is a sequence's state
+  DifferentialAttention     two rotated softmax maps per head over the same values, a1 - lambda a2, unit-normed, with one
+                            gate number per head; visibility within chunks of the sequence or causal
+  GeneralDeltaMixer         generalised delta rule: channel-wise decay, removal along the unit key at a rate per channel
 
 Layers whose weights a model runs several times per step (a looped stack) keep one cache / state per pass ("lane"): their
 forward takes the lane's number.
@@ -356,11 +363,11 @@ class BiasedAttention(nn.Module):
 
 
 class GatedDenseMLP(nn.Module):
-    def __init__(self, width: int, ff: int, act: str = "gelu_tanh"):
+    def __init__(self, width: int, ff: int, act: str = "gelu_tanh", bias: bool = True):
         super().__init__()
         self.act = _ACTS[act]
         self.gate, self.up, self.down = _matrix(ff, width), _matrix(ff, width), _matrix(width, ff)
-        self.gate_b, self.up_b, self.down_b = _vector(ff), _vector(ff), _vector(width)
+        self.gate_b, self.up_b, self.down_b = (_vector(ff), _vector(ff), _vector(width)) if bias else (None, None, None)
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         a = ops.gemm_any_act(h, self.gate, bias=self.gate_b, act=self.act, w2=self.up, bias2=self.up_b)
@@ -691,3 +698,151 @@ class InputWeightedSparseMLP(nn.Module):
                                      offsets, P, None, P)
         y = ops.gemm_any_grouped(a, None, self.down, None, offsets, P, pair_index, P)
         return ops.moe_combine_shared(y, ids, None, h.shape[1])
+
+
+# ---------------------------------------------------------------------------------------------------------------------
+# families with several residual streams: differential attention heads, the generalised delta rule
+# ---------------------------------------------------------------------------------------------------------------------
+class TokenShift(nn.Module):
+    """h_t <- h_t + (h_{t-1} - h_t) * weight per channel, with h_{t-1} as it was before its own shift (zeros before position
+    0).  The last h of a sequence lives in its state slot, one [slots, width] per lane."""
+
+    def __init__(self, width: int):
+        super().__init__()
+        self.weight = _vector(width)
+        self.state = []
+
+    def state_shape(self, n_slots: int):
+        return (n_slots, self.weight.shape[0])
+
+
+class StreamCoefficients(nn.Module):
+    """What one sublayer does with the streams: reads sum_s read[s] X_s, leaves X_t <- sum_s mix[s, t] X_s + write[t] y."""
+
+    def __init__(self, streams: int):
+        super().__init__()
+        self.read, self.write = _vector(streams, 1.0), _vector(streams, 1.0)
+        self.mix = nn.Parameter(torch.eye(streams, dtype=torch.float32), requires_grad=False)
+
+
+class StreamResidual:
+    """The residual streams of one step, [rows, streams, width] fp32, all the embedding row at the start.  A sublayer
+    boundary - the last sublayer's output into the streams, the next one's input out of them, its norm over `groups` parts of
+    the channels and its token shift - is one launch (one more advances the shift's state when a sequence brings several
+    rows)."""
+
+    def __init__(self, embedded: torch.Tensor, streams: int, groups: int, eps: float):
+        self.src = embedded.unsqueeze(1).expand(-1, streams, -1)   # (until the first sublayer has left its output)
+        self.own = self.spare = None      # buffers of the streams
+        self.groups, self.eps = groups, eps
+        self.pending = None               # (output, coefficients) of the last sublayer, not in the streams yet
+
+    def leave(self, y: torch.Tensor, coef: StreamCoefficients) -> None:
+        assert self.pending is None
+        self.pending = (y, coef)
+
+    def _boundary(self, read, norm_w, store: bool, shift: TokenShift | None = None, lane: int = 0) -> torch.Tensor:
+        ctx, extra, moves = get_context(), {}, False
+        if shift is not None:
+            extra = dict(shift=shift.weight, shift_state=shift.state[lane], cu_q=ctx.cu_seqlens_q, kv_lens=ctx.kv_lens,
+                         slot_ids=ctx.state_slots, max_rows_per_seq=ctx.max_seqlen_q)
+            moves = ctx.max_seqlen_q > 1   # a row also reads the old streams of the row before it: not in place
+        y, coef = self.pending or (None, None)
+        dst = None
+        if y is not None and store:
+            dst = self.spare if moves else self.own
+            if self.own is None or dst is None:
+                dst = torch.empty(self.src.shape, dtype=torch.float32, device=self.src.device)
+        h = ops.stream_mix(self.src, dst, y, *((coef.mix, coef.write) if coef is not None else (None, None)), read, norm_w,
+                           self.groups, self.eps, **extra)
+        if dst is not None:
+            if dst is not self.own:
+                self.own, self.spare = dst, self.own
+            self.src = dst
+        self.pending = None if dst is not None or y is None else self.pending
+        return h
+
+    def read(self, coef: StreamCoefficients, norm_w: torch.Tensor, shift: TokenShift | None = None, lane: int = 0) -> torch.Tensor:
+        """what the next sublayer reads: the normed (and shifted) weighted sum of the streams"""
+        return self._boundary(coef.read, norm_w, True, shift, lane)
+
+    def total(self, store: bool = False) -> torch.Tensor:
+        """the sum of the streams; store: the streams themselves are brought up to date too"""
+        return self._boundary(None, None, store)
+
+
+class DifferentialAttention(nn.Module):
+    """q [heads][2][dim], k [kv_heads][2][dim], v [kv_heads][vdim] = W h + b; both maps of q and k rotated (pairs i,
+    i + rot_dims / 2); map m of a head: a_m = softmax(scale q_m . k_m) v over the visible keys; lambda = exp(lq1 . lk1) -
+    exp(lq2 . lk2) + diff; o = rms-unit(a_1 - lambda a_2) (1 - diff) sigmoid(W_g h)_head; out = W_o o + b.  chunk > 0: only
+    keys of a position's own chunk are visible.
+
+    The maps are key heads of their own (2 kv_heads of them) that share kv_heads value heads: with the query rows stored
+    [kv head][map][query head of the group], the paged attention's usual grouping reads the right map and the right value
+    head for every query row, and a1, a2 of a head's group lie side by side."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, chunk: int, scale: float, diff: float,
+                 eps: float, rot_dims: int, rot_base: float):
+        super().__init__()
+        assert heads % kv_heads == 0 and 0 <= rot_dims <= dim and rot_dims % 2 == 0
+        self.H, self.G, self.D, self.Dv, self.chunk, self.scale = heads, kv_heads, dim, vdim, chunk, scale
+        self.diff, self.eps, self.rot_dims = diff, eps, rot_dims
+        self.register_buffer("inv_freq", rotary_inv_freq(rot_dims, rot_base), persistent=False)
+        self.qkvg = MergedRows(width, {"q": heads * 2 * dim, "k": kv_heads * 2 * dim, "v": kv_heads * vdim, "g": heads}, bias=True)
+        self.qkvg.weight.weight_loader = self.qkvg.bias.weight_loader = self._load
+        # lq1, lk1, lq2, lk2
+        self.lam = nn.Parameter(torch.zeros(4, dim, dtype=torch.float32), requires_grad=False)
+        self.lam.weight_loader = lambda param, tensor, row: param.data[row].copy_(tensor)
+        self.o, self.o_b = _matrix(width, heads * vdim), _vector(width)
+        self.k_cache, self.v_cache = [], []   # one per lane
+
+    def _load(self, param, tensor, shard):
+        if shard == "q":
+            t = tensor.view(self.G, self.H // self.G, 2, self.D, *tensor.shape[1:])
+            tensor = t.transpose(1, 2).reshape(tensor.shape)
+        self.qkvg._load(param, tensor, shard)
+
+    def cache_shapes(self, num_blocks: int, block_size: int):
+        return (num_blocks, 2 * self.G, block_size, self.D), (num_blocks, self.G, block_size, self.Dv)
+
+    def forward(self, h: torch.Tensor, lane: int = 0) -> torch.Tensor:
+        ctx, m = get_context(), self.qkvg
+        H, G, D, Dv = self.H, self.G, self.D, self.Dv
+        kc, vc = self.k_cache[lane], self.v_cache[lane]
+        y = m(h)
+        ops.rotary_store(y, m.offsets["q"][0], m.offsets["k"][0], m.offsets["v"][0], 2 * H, 2 * G, D, self.rot_dims,
+                         _C.ROT_HALVES, self.inv_freq, 1.0, False, self.eps, 1.0, ctx.cu_seqlens_q, ctx.kv_lens, kc, vc,
+                         ctx.slot_mapping, ctx.block_size)
+        o = ops.paged_attention_f32(m.cols(y, "q"), kc, vc, Dv, ctx.block_tables, ctx.cu_seqlens_q, ctx.kv_lens, 2 * H, 2 * G, D,
+                                    Dv, ctx.block_size, CAUSAL, self.scale, value_heads=G, chunk=self.chunk)
+        o = ops.diff_heads(o, self.lam, self.diff, self.eps, m.cols(y, "g"), H, G, Dv)
+        return ops.gemm_any_act(o, self.o, bias=self.o_b)
+
+
+class GeneralDeltaMixer(nn.Module):
+    """r, k, v = W h; w = exp(-exp(-1/2) sigmoid(W_2 tanh(W_1 h) + w0)), a = sigmoid(W_a h + b) per head and channel;
+    u = k / sqrt(sum k^2 + 1e-6); S <- diag(w) S - (a u) (u^T S) + k v^T, o = S^T r (fp32 state per sequence slot and lane);
+    out = W_o (rms-unit(o) per head * norm * sigmoid(W_g h)).  The six projections of h are one product whose epilogue
+    applies the sigmoid of a and the tanh of the low-rank path; the decay comes out of the second product's epilogue."""
+
+    def __init__(self, width: int, heads: int, dim: int, rank: int, eps: float):
+        super().__init__()
+        n = heads * dim
+        self.H, self.D, self.eps = heads, dim, eps
+        self.proj = MergedRows(width, {"r": n, "k": n, "v": n, "g": n, "a": n, "w1": rank}, bias=True)
+        self.w2, self.w0, self.norm = _matrix(n, rank), _vector(n), _vector(n, 1.0)
+        self.o = _matrix(width, n)
+        self.state = []   # one per lane
+
+    def state_shape(self, n_slots: int):
+        return (n_slots, ops.general_delta_state_elems(self.H, self.D, self.D))
+
+    def forward(self, h: torch.Tensor, lane: int = 0) -> torch.Tensor:
+        ctx, m = get_context(), self.proj
+        off = {name: o for name, (o, _) in m.offsets.items()}
+        y = ops.gemm_any_segments(h, m.weight, m.bias, _C.ACT_SIGMOID, off["a"], _C.ACT_TANH, off["w1"])
+        w = ops.gemm_any_act(m.cols(y, "w1"), self.w2, bias=self.w0, act=_C.ACT_DECAY)
+        o = ops.general_delta(y, off["r"], off["k"], off["v"], off["a"], w, self.state[lane], ctx.cu_seqlens_q, ctx.kv_lens,
+                              ctx.state_slots, self.H, self.D, self.D)
+        ops.head_norm_gate(o, m.cols(y, "g"), _C.ACT_SIGMOID, self.norm, self.H, self.D, self.eps)
+        return ops.gemm_any(o, self.o)

@@ -5,6 +5,7 @@ qwen3.py:70-72 switches between q/k norm and qkv bias), Llama (models/llama.py) 
 from nanovllm.models.felolorn import FelolornConfig, FelolornForCausalLM
 from nanovllm.models.gazutar import GazutarConfig, GazutarForCausalLM
 from nanovllm.models.llama import LlamaForCausalLM
+from nanovllm.models.munizen import MunizenConfig, MunizenForCausalLM
 from nanovllm.models.qwen3 import Qwen3ForCausalLM
 from nanovllm.models.qwen3_moe import Qwen3MoeForCausalLM
 from nanovllm.models.sanevik import SanevikConfig, SanevikForCausalLM
@@ -19,6 +20,7 @@ model_dict = {
     "Zedirax": ZediraxForCausalLM,
     "Felolorn": FelolornForCausalLM,
     "Sanevik": SanevikForCausalLM,
+    "Munizen": MunizenForCausalLM,
 }
 
 # designs whose config.json is not a transformers configuration: {"architecture": <name>, ...} -> the reader of it
@@ -27,6 +29,7 @@ native_configs = {
     "Zedirax": ZediraxConfig,
     "Felolorn": FelolornConfig,
     "Sanevik": SanevikConfig,
+    "Munizen": MunizenConfig,
 }
 
 

@@ -33,9 +33,10 @@ from torch import nn
 from nanovllm import ops
 from nanovllm.layers.seqmix import (CAUSAL, InputWeightedSparseMLP, ParallelMixers, Retention, RotaryWindowAttention,
                                     SinkAttentionMixer, _vector)
+from nanovllm.models.looped import LoopedLayers
 
 
-class SanevikConfig:
+class SanevikConfig(LoopedLayers):
     """config.json of this design with the attribute names the engine reads from a configuration object."""
     architectures = ["Sanevik"]
     model_type = "sanevik"
@@ -49,26 +50,8 @@ class SanevikConfig:
         self.layers = raw["layers"]
         self.num_hidden_layers = len(self.layers)
         self.norm_eps = float(raw["norm"]["eps"])
-        loop = raw.get("loop")
-        n = len(self.layers)
-        self.loop_start, self.loop_stop, self.loop_times = (int(loop["start"]), int(loop["stop"]), int(loop["times"])) \
-            if loop else (0, 0, 0)
-        assert 0 <= self.loop_start <= self.loop_stop <= n and (not loop or self.loop_times >= 1), loop
+        self.read_loop(raw.get("loop"), len(self.layers))
         self.torch_dtype = dtype
-
-    @property
-    def layer_runs(self):
-        """[(layer, lane, pass number on a pass's first layer or None)] in execution order"""
-        a, b, n = self.loop_start, self.loop_stop, len(self.layers)
-        if not self.loop_times or a == b:
-            return [(i, 0, None) for i in range(n)]
-        runs = [(i, 0, None) for i in range(a)]
-        for t in range(self.loop_times):
-            runs += [(i, t, t if i == a else None) for i in range(a, b)]
-        return runs + [(i, 0, None) for i in range(b, n)]
-
-    def lanes_of(self, i: int) -> int:
-        return self.loop_times if self.loop_times and self.loop_start <= i < self.loop_stop else 1
 
     @classmethod
     def from_dir(cls, path: str, dtype: str = "bfloat16") -> "SanevikConfig":

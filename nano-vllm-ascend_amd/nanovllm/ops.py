@@ -1204,10 +1204,10 @@ def gemm_any_batched(x, x_batch: int, w, out, out_batch: int, gate=None, gate_ba
 def paged_attention_f32(q, k_cache, v_cache, ldv: int, block_tables, cu_q, kv_lens, H: int, G: int, D: int, Dv: int,
                         block_size: int, window: int, scale: float, bias_kind: int = _C.BIAS_NONE, bias_p1=None, bias_p2=None,
                         gate=None, sink=None, softcap: float = 0.0, value_heads: int | None = None,
-                        v_offset: int = 0, out=None) -> torch.Tensor:
+                        v_offset: int = 0, chunk: int = 0, out=None) -> torch.Tensor:
     """Paged causal attention over fp32 queries; see mi_paged_attention_ext (bias kinds, values inside the key rows, a
     sink logit per head in the softmax's denominator, capped scores, fewer and wider value heads than key heads with the
-    value rows read from column v_offset on)."""
+    value rows read from column v_offset on, visibility within chunks of `chunk` positions)."""
     require_gpu(q, k_cache, v_cache, block_tables, cu_q, kv_lens)
     _f32(q, gate, bias_p1, bias_p2, sink)
     assert sink is None or (sink.numel() == H and sink.is_contiguous())
@@ -1226,7 +1226,7 @@ def paged_attention_f32(q, k_cache, v_cache, ldv: int, block_tables, cu_q, kv_le
     check(lib.mi_paged_attention_ext(ptr(q), q.stride(0), ptr(k_cache), ptr(v_cache) + v_offset * v_cache.element_size(),
                                      int(ldv), _dt(k_cache),
                                      ptr(block_tables), block_tables.shape[1], ptr(cu_q), ptr(kv_lens), n_seqs, rows, H, G,
-                                     D, Dv, block_size, int(min(window, 2 ** 31 - 1)), float(scale), int(bias_kind),
+                                     D, Dv, block_size, int(min(window, 2 ** 31 - 1)), int(chunk), float(scale), int(bias_kind),
                                      ptr(bias_p1), ptr(bias_p2), ptr(sink), float(softcap),
                                      int(G if value_heads is None else value_heads), ptr(gate),
                                      gate.stride(0) if gate is not None else 0,
@@ -1458,11 +1458,99 @@ def head_mix(o, talk, H: int, G: int, Dv: int, c0: int, n_chunk: int, out, out_s
 
 
 def head_norm_gate(out, gate_pre, gate_act: int, norm_w, H: int, Dv: int, eps: float, out_scale: float = 1.0) -> None:
-    """out[:, h] <- out_scale * out[:, h] / rms (* norm_w) (* act(gate_pre[:, h])) per head, in place."""
+    """out[:, h] <- out_scale * out[:, h] / rms (* norm_w) (* act(gate_pre[:, h])) per head, in place; norm_w [Dv] (every
+    head's) or [H * Dv]."""
     require_gpu(out)
     _f32(out, gate_pre, norm_w)
     assert out.shape[1] >= H * Dv and (gate_pre is None or (gate_pre.shape[0] == out.shape[0] and gate_pre.shape[1] >= H * Dv))
-    assert norm_w is None or norm_w.numel() == Dv
+    assert norm_w is None or (norm_w.is_contiguous() and norm_w.numel() in (Dv, H * Dv))
+    stride = Dv if norm_w is not None and norm_w.numel() == H * Dv else 0
     check(lib.mi_head_norm_gate(ptr(out), out.stride(0), ptr(gate_pre), gate_pre.stride(0) if gate_pre is not None else 0,
-                                int(gate_act), ptr(norm_w), float(out_scale), out.shape[0], H, Dv, float(eps), stream()),
+                                int(gate_act), ptr(norm_w), stride, float(out_scale), out.shape[0], H, Dv, float(eps), stream()),
           "mi_head_norm_gate")
+
+
+# ---- families with several residual streams, differential heads, the generalised delta rule (csrc/stream_delta.hip)
+def gemm_any_segments(x, w, bias, act: int, act_from: int, act2: int | None = None, act2_from: int | None = None,
+                      exact: bool = False) -> torch.Tensor:
+    """x w^T + bias; features from act_from on through `act`, those from act2_from on through `act2` instead."""
+    require_gpu(x, w)
+    _f32(x, bias)
+    assert x.dim() == 2 and w.dim() == 2 and w.is_contiguous() and x.shape[1] == w.shape[1], (x.shape, w.shape)
+    M, K = x.shape
+    N = w.shape[0]
+    assert bias is None or bias.numel() == N
+    out = torch.empty((M, N), dtype=_F32, device=x.device)
+    check(lib.mi_gemm_any_segments(ptr(x), x.stride(0) if M > 1 else K, ptr(w), _dt(w), ptr(bias), int(act), int(act_from),
+                                   int(act if act2 is None else act2), int(N if act2_from is None else act2_from), ptr(out), N,
+                                   M, N, K, int(exact), stream()), "mi_gemm_any_segments")
+    return out
+
+
+def stream_mix(src, dst, y, mix, out_coef, in_coef, norm_w, groups: int, eps: float, shift=None, shift_state=None, cu_q=None,
+               kv_lens=None, slot_ids=None, max_rows_per_seq: int = 1) -> torch.Tensor:
+    """One sublayer boundary of a stream-residual model (see mi_stream_mix).  src: [rows, streams, width], or [rows, width]
+    expanded to it (every stream the same row); dst: [rows, streams, width] or None; returns h [rows, width]."""
+    require_gpu(src, dst, y)
+    _f32(src, dst, y, mix, out_coef, in_coef, norm_w, shift, shift_state)
+    _i32(cu_q, kv_lens, slot_ids)
+    rows, n, width = src.shape
+    assert dst is None or dst.shape == src.shape
+    assert y is None or (y.shape == (rows, width) and mix.shape == (n, n) and mix.is_contiguous() and out_coef.numel() == n)
+    assert in_coef is None or in_coef.numel() == n
+    assert norm_w is None or norm_w.numel() == width
+    h = torch.empty((rows, width), dtype=_F32, device=src.device)
+    n_seqs, carry = 0, None
+    if shift is not None:
+        n_seqs = kv_lens.numel()
+        assert shift.numel() == width and shift_state.is_contiguous() and shift_state.shape[1] == width and cu_q.numel() == n_seqs + 1
+        if max_rows_per_seq > 1:
+            carry = torch.empty((n_seqs, width), dtype=_F32, device=src.device)
+    # (one row: torch reports arbitrary strides for a dimension of size 1)
+    ld = lambda t, least: 0 if t is None else t.stride(0) if rows > 1 else max(t.stride(0), least)
+    ss = src.stride(1) if n > 1 else width
+    ds = width if dst is None or n == 1 else dst.stride(1)
+    check(lib.mi_stream_mix(ptr(src), ld(src, ss * (n - 1) + width), ss, ptr(dst), ld(dst, ds * (n - 1) + width), ds, n, ptr(y),
+                            ld(y, width), ptr(mix), ptr(out_coef), ptr(in_coef), ptr(norm_w), int(groups), float(eps), ptr(shift),
+                            ptr(shift_state), ptr(carry), ptr(cu_q), ptr(kv_lens), ptr(slot_ids), n_seqs, int(max_rows_per_seq),
+                            ptr(h), width, rows, width, stream()), "mi_stream_mix")
+    return h
+
+
+def diff_heads(o, lam, diff: float, eps: float, gate, H: int, G: int, Dv: int) -> torch.Tensor:
+    """o [rows, G * 2 * (H / G) * Dv]: the read-outs of both maps; lam [4, D]; gate [rows, >= H] or None -> [rows, H * Dv]."""
+    require_gpu(o, lam)
+    _f32(o, lam, gate)
+    rows = o.shape[0]
+    assert o.shape[1] == 2 * H * Dv and lam.dim() == 2 and lam.shape[0] == 4 and lam.is_contiguous()
+    assert gate is None or (gate.shape[0] == rows and gate.shape[1] >= H)
+    out = torch.empty((rows, H * Dv), dtype=_F32, device=o.device)
+    check(lib.mi_diff_heads(ptr(o), max(o.stride(0), 2 * H * Dv), ptr(lam), lam.shape[1], float(diff), float(eps), ptr(gate),
+                            max(gate.stride(0), H) if gate is not None else 0, ptr(out), H * Dv, rows, H, G, Dv, stream()),
+          "mi_diff_heads")
+    return out
+
+
+def general_delta_state_elems(H: int, D: int, Dv: int) -> int:
+    """Floats of state per sequence slot (the kernel keeps it in its own thread-order layout)."""
+    n = lib.mi_general_delta_state_elems(H, D, Dv)
+    if n < 0:
+        raise _C.MiError(f"generalised delta rule: {D} key channels per head are beyond the compiled kernels (<= 256)")
+    return n
+
+
+def general_delta(proj, r_off: int, k_off: int, v_off: int, a_off: int, w_decay, state, cu_q, kv_lens, slot_ids, H: int, D: int,
+                  Dv: int) -> torch.Tensor:
+    """S <- diag(w) S - (a u)(u^T S) + k v^T, o = S^T r per head over the step's rows (see mi_general_delta); the raw
+    read-out [rows, H * Dv]."""
+    require_gpu(proj, w_decay, state)
+    _f32(proj, w_decay, state)
+    _i32(cu_q, kv_lens, slot_ids)
+    rows = proj.shape[0]
+    assert state.is_contiguous() and state.shape[1] == general_delta_state_elems(H, D, Dv), state.shape
+    assert w_decay.shape[0] == rows and w_decay.shape[1] >= H * D and cu_q.numel() == kv_lens.numel() + 1
+    out = torch.empty((rows, H * Dv), dtype=_F32, device=proj.device)
+    check(lib.mi_general_delta(ptr(proj), max(proj.stride(0), proj.shape[1]), r_off, k_off, v_off, a_off, ptr(w_decay),
+                               max(w_decay.stride(0), H * D), ptr(state), ptr(cu_q), ptr(kv_lens), ptr(slot_ids), kv_lens.numel(),
+                               rows, H, D, Dv, ptr(out), H * Dv, stream()), "mi_general_delta")
+    return out
