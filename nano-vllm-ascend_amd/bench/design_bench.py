@@ -1,5 +1,5 @@
 """Prefill and decode throughput of a model design beside the framework's closest existing model at equal size
-(`python bench.py --design gazutar | zedirax | felolorn | sanevik`): random weights, layer sizes that resemble a real model's, both models through the same
+(`python bench.py --design gazutar | zedirax | felolorn | sanevik | munizen`): random weights, layer sizes that resemble a real model's, both models through the same
 engine entry points (add_request / step), each served the way the framework serves it (Qwen3-MoE: captured prefill and
 decode steps; Gazutar: what ModelRunner reports in `served_as`).
 
@@ -153,6 +153,36 @@ def sanevik_decode_weight_bytes(cfg: dict, batch: int) -> float:
     return 2.0 * (n + cfg["vocab"] * W)
 
 
+def munizen_config(s: dict) -> dict:
+    """Generalised delta rule / differential attention in chunks of the other models' window, alternating; the last two
+    layers run twice (six layer runs per step, each with pages and state of its own); four residual streams, norms in two
+    groups.  A head's two maps have half the head size each, so the projections are as wide as the others'; the dense
+    feed-forward is as wide as the experts a token visits in the others."""
+    W, D, H, G = s["width"], s["dim"], s["heads"], s["kv_heads"]
+    att = {"type": "attention",
+           "mixer": {"heads": H, "kv_heads": G, "dim": D // 2, "vdim": D, "mask": {"size": s["window"]}, "scale": (D // 2) ** -0.5,
+                     "diff": 0.6, "rot": {"base": 10000.0, "dims": D // 2}}}
+    rec = {"type": "general_delta", "mixer": {"heads": H, "dim": D, "rank": W // 16}}
+    ff = {"kind": "dense", "ff": s["top"] * s["ff"]}
+    n = s["layers"]
+    return {"architecture": "Munizen", "vocab": s["vocab"], "width": W, "streams": 4, "norm": {"eps": 1e-6, "groups": 2},
+            "loop": {"start": n - 2, "stop": n, "times": 2},
+            "layers": [dict((rec, att)[i % 2], mlp=ff) for i in range(n)]}
+
+
+def munizen_decode_weight_bytes(cfg: dict) -> float:
+    """bf16 weight bytes a decode step streams: every projection once per RUN of a layer, the head."""
+    W, n, loop = cfg["width"], 0, cfg["loop"]
+    for i, l in enumerate(cfg["layers"]):
+        m = l["mixer"]
+        if l["type"] == "attention":
+            mix = W * (2 * (m["heads"] + m["kv_heads"]) * m["dim"] + m["kv_heads"] * m["vdim"] + m["heads"] * (1 + m["vdim"]))
+        else:
+            mix = W * (6 * m["heads"] * m["dim"] + m["rank"]) + m["rank"] * m["heads"] * m["dim"]
+        n += (mix + 3 * W * l["mlp"]["ff"]) * (loop["times"] if loop["start"] <= i < loop["stop"] else 1)
+    return 2.0 * (n + cfg["vocab"] * W)
+
+
 def qwen3_moe_config(s: dict) -> dict:
     return dict(architectures=["Qwen3MoeForCausalLM"], model_type="qwen3_moe", hidden_size=s["width"],
                 num_hidden_layers=s["layers"], num_attention_heads=s["heads"], num_key_value_heads=s["kv_heads"],
@@ -232,6 +262,8 @@ def main(args) -> dict:
         return main_felolorn(args, batch, prompt_len)
     if design == "sanevik":
         return main_sanevik(args, batch, prompt_len)
+    if design == "munizen":
+        return main_munizen(args, batch, prompt_len)
     out = {"metric": "design_throughput", "design": "gazutar", "closest_model": "Qwen3MoeForCausalLM", "unit": "tokens/s",
            "dtype": "bf16", "data": "synthetic (random weights, random prompts)", "n_gpus": 1, "steps": args.steps,
            "warmup": args.warmup, "batch": batch, "prompt_len": prompt_len, "sizes": {}}
@@ -351,6 +383,40 @@ def main_sanevik(args, batch: int, prompt_len: int) -> dict:
                 entry["sanevik_vs_" + other] = {k: entry["sanevik"][k] / entry[other][k] for k in ("prefill_tok_s", "decode_tok_s")}
                 entry["sanevik_vs_" + other + "_per_layer_run"] = {
                     k: v * entry["sanevik"]["layer_runs"] / entry[other]["layer_runs"] for k, v in entry["sanevik_vs_" + other].items()}
+        out["sizes"][name] = entry
+    print(json.dumps(out), flush=True)
+    return out
+
+
+def main_munizen(args, batch: int, prompt_len: int) -> dict:
+    """Munizen beside Gazutar - the closest existing model: the same row-step engine path, fp32 residual, a delta rule with a
+    decay per key channel alternating with windowed attention - at equal width, depth, heads and vocabulary; Sanevik (looped,
+    rotated heads) rides along (`--design-models` picks).  `layer_runs` counts a looped layer once per pass."""
+    out = {"metric": "design_throughput", "design": "munizen", "closest_model": "Gazutar", "unit": "tokens/s",
+           "dtype": "bf16", "data": "synthetic (random weights, random prompts)", "n_gpus": 1, "steps": args.steps,
+           "warmup": args.warmup, "batch": batch, "prompt_len": prompt_len, "sizes": {}}
+    only_sizes = [x for x in getattr(args, "design_sizes", "").split(",") if x]
+    only_models = [x for x in getattr(args, "design_models", "").split(",") if x] or ["munizen", "gazutar", "sanevik"]
+    for name, s in SIZES.items():
+        if only_sizes and name not in only_sizes:
+            continue
+        entry = {"shape": s}
+        mc, sc = munizen_config(s), sanevik_config(s)
+        for label, cfg, wb, runs in (("munizen", mc, munizen_decode_weight_bytes(mc), s["layers"] + 2),
+                                     ("gazutar", gazutar_config(s), decode_weight_bytes(s, batch, True), s["layers"]),
+                                     ("sanevik", sc, sanevik_decode_weight_bytes(sc, batch), s["layers"] + 2)):
+            if label not in only_models:
+                continue
+            r = run_model(cfg, batch, prompt_len, args.steps, args.warmup)
+            r["layer_runs"] = runs
+            r["decode_weight_bytes"] = wb
+            r["decode_weight_roofline_frac"] = wb / (r["ms_per_decode_step"] * 1e-3) / HBM_BYTES_PER_S
+            entry[label] = r
+        for other in ("gazutar", "sanevik"):
+            if "munizen" in entry and other in entry:
+                entry["munizen_vs_" + other] = {k: entry["munizen"][k] / entry[other][k] for k in ("prefill_tok_s", "decode_tok_s")}
+                entry["munizen_vs_" + other + "_per_layer_run"] = {
+                    k: v * entry["munizen"]["layer_runs"] / entry[other]["layer_runs"] for k, v in entry["munizen_vs_" + other].items()}
         out["sizes"][name] = entry
     print(json.dumps(out), flush=True)
     return out

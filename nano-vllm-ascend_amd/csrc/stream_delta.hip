@@ -226,26 +226,35 @@ __global__ __launch_bounds__(256) void diff_heads_kernel(const float* __restrict
 // column.  The dot for row t + 1 is summed while row t's new column is formed: ONE pass over the state per row, with two
 // independent sums (read-out and next dot) whose cross-lane ends overlap - a two-pass walk waits for the dot before it may
 // touch the state.
-// A workgroup = 32 value columns of one (sequence, head); sixteen lanes share CPL columns, lane r keeping the key channels
-// (16 jj + r) * 4 + e of them in registers for the whole walk over the step's rows (each LDS vector of a row read once for
-// CPL columns).  ROWS rows at a time go through LDS, fetched one batch ahead and turned into r, u, w, a and |k| v on the
-// way: the staging lanes of a row sum its k^2 among themselves.  State in thread order, 16-byte pieces.
-constexpr int kGdCols = 32, kGdLanes = 16;
+// A workgroup = 32 value columns of one (sequence, head); LANES lanes share CPL columns, lane r keeping the key channels
+// (LANES jj + r) * 4 + e of them in registers for the whole walk over the step's rows.  ROWS rows at a time go through LDS,
+// fetched one batch ahead and turned into r, u, w, a and |k| v on the way: the staging lanes of a row sum its k^2 among
+// themselves.  A full batch is walked by unrolled code, so that the LDS reads of later rows run ahead of the walk.  (8
+// sequences x 1024 rows x 8 heads x 128 channels, 16 lanes: one column per lane group 285 us, two 435 us, 8 lanes 350 us; not
+// unrolled 430 us.)  State in thread order, 16-byte pieces.
+constexpr int kGdCols = 32;
 
-template <int DR, int CPL, int ROWS>  // DR: key channels per lane
-__global__ __launch_bounds__(kGdLanes* kGdCols / CPL) void general_delta_kernel(
+template <int LANES>
+__device__ __forceinline__ float lanes_sum(float v) {  // over the LANES neighbours that share a column
+  v = xor_sum<4>(xor_sum<2>(xor_sum<1>(v)));
+  if constexpr (LANES == 16) v = xor_sum<8>(v);
+  return v;
+}
+
+template <int LANES, int DR, int CPL, int ROWS>  // DR: key channels per lane
+__global__ __launch_bounds__(LANES* kGdCols / CPL) void general_delta_kernel(
     const float* __restrict__ proj, int64_t ld, int r_off, int k_off, int v_off, int a_off, const float* __restrict__ wdec,
     int64_t ldw, float* __restrict__ state, const int32_t* __restrict__ cu_q, const int32_t* __restrict__ kv_lens,
     const int32_t* __restrict__ slot_ids, int H, int D, int Dv, float* __restrict__ out, int64_t ldo) {
-  constexpr int NT = kGdLanes * kGdCols / CPL, DP = kGdLanes * DR, SL = NT / ROWS, PE = DP / SL, JJ = DR / 4;
-  static_assert(SL * ROWS == NT && (SL == 16 || SL == 32) && DP % SL == 0 && kGdCols % SL == 0, "staging shape");
+  constexpr int NT = LANES * kGdCols / CPL, DP = LANES * DR, SL = NT / ROWS, PE = DP / SL, JJ = DR / 4;
+  static_assert(SL * ROWS == NT && (SL == 8 || SL == 16 || SL == 32) && DP % SL == 0 && kGdCols % SL == 0, "staging shape");
   __shared__ __attribute__((aligned(16))) float rs[ROWS][DP];
   __shared__ __attribute__((aligned(16))) float us[ROWS][DP];
   __shared__ __attribute__((aligned(16))) float ws[ROWS][DP];
   __shared__ __attribute__((aligned(16))) float as[ROWS][DP];
   __shared__ float vs[ROWS][kGdCols];
   const int s = blockIdx.x, h = blockIdx.y, cb = blockIdx.z;
-  const int tid = threadIdx.x, r = tid & (kGdLanes - 1), cg = tid / kGdLanes;
+  const int tid = threadIdx.x, r = tid & (LANES - 1), cg = tid / LANES;
   const int r0 = cu_q[s], n = cu_q[s + 1] - r0;
   if (n == 0) return;
   const int start = kv_lens[s] - n;
@@ -286,7 +295,7 @@ __global__ __launch_bounds__(kGdLanes* kGdCols / CPL) void general_delta_kernel(
     float sq = 0.f;
 #pragma unroll
     for (int m = 0; m < PE; ++m) sq = fmaf(fk[m], fk[m], sq);
-    sq = xor_sum<8>(xor_sum<4>(xor_sum<2>(xor_sum<1>(sq))));
+    sq = lanes_sum<(SL >= 16 ? 16 : 8)>(sq);
     if constexpr (SL == 32) sq = xor_sum<16>(sq);
     const float len = sqrtf(sq + 1e-6f), inv = 1.f / len;
     __syncthreads();  // the previous rows' vectors have been consumed
@@ -300,56 +309,56 @@ __global__ __launch_bounds__(kGdLanes* kGdCols / CPL) void general_delta_kernel(
     __syncthreads();
     if (c0 + ROWS < n) fetch(c0 + ROWS);
     const int nt = min(ROWS, n - c0);
-    // the batch's first dot: a pass of its own
+    auto load = [&](const float(&m)[ROWS][DP], int t, float(&x)[DR]) {
+#pragma unroll
+      for (int jj = 0; jj < JJ; ++jj) {
+        const float4 q = reinterpret_cast<const float4*>(m[t])[jj * LANES + r];
+        x[jj * 4 + 0] = q.x, x[jj * 4 + 1] = q.y, x[jj * 4 + 2] = q.z, x[jj * 4 + 3] = q.w;
+      }
+    };
     float u[DR], dot[CPL];
+    load(us, 0, u);
 #pragma unroll
-    for (int jj = 0; jj < JJ; ++jj) {
-      const float4 x = reinterpret_cast<const float4*>(us[0])[jj * kGdLanes + r];
-      u[jj * 4 + 0] = x.x, u[jj * 4 + 1] = x.y, u[jj * 4 + 2] = x.z, u[jj * 4 + 3] = x.w;
-    }
-#pragma unroll
-    for (int cc = 0; cc < CPL; ++cc) {
+    for (int cc = 0; cc < CPL; ++cc) {  // the batch's first dot: a pass of its own
       float d0 = 0.f, d1 = 0.f;
 #pragma unroll
       for (int e = 0; e < DR; e += 2) d0 = fmaf(u[e], st[cc][e], d0), d1 = fmaf(u[e + 1], st[cc][e + 1], d1);
-      dot[cc] = xor_sum<8>(xor_sum<4>(xor_sum<2>(xor_sum<1>(d0 + d1))));
+      dot[cc] = lanes_sum<LANES>(d0 + d1);
     }
-    for (int t = 0; t < nt; ++t) {
-      const float4* r4 = reinterpret_cast<const float4*>(rs[t]);
-      const float4* w4 = reinterpret_cast<const float4*>(ws[t]);
-      const float4* a4 = reinterpret_cast<const float4*>(as[t]);
-      const float4* u4 = reinterpret_cast<const float4*>(us[min(t + 1, nt - 1)]);
-      float v[CPL], o0[CPL], o1[CPL], d0[CPL], d1[CPL];
-#pragma unroll
-      for (int cc = 0; cc < CPL; ++cc) v[cc] = vs[t][cg * CPL + cc], o0[cc] = o1[cc] = d0[cc] = d1[cc] = 0.f;
-#pragma unroll
-      for (int jj = 0; jj < JJ; ++jj) {
-        const float4 rv = r4[jj * kGdLanes + r], wv = w4[jj * kGdLanes + r], av = a4[jj * kGdLanes + r],
-                     un = u4[jj * kGdLanes + r];
-        const float rr[4] = {rv.x, rv.y, rv.z, rv.w}, ww[4] = {wv.x, wv.y, wv.z, wv.w}, aa[4] = {av.x, av.y, av.z, av.w},
-                    nn[4] = {un.x, un.y, un.z, un.w};
-#pragma unroll
-        for (int cc = 0; cc < CPL; ++cc)
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            float& S = st[cc][jj * 4 + e];
-            S = fmaf(ww[e], S, u[jj * 4 + e] * fmaf(-aa[e], dot[cc], v[cc]));
-            float& o = e & 1 ? o1[cc] : o0[cc];
-            float& d = e & 1 ? d1[cc] : d0[cc];
-            o = fmaf(rr[e], S, o);
-            d = fmaf(nn[e], S, d);
-          }
-#pragma unroll
-        for (int e = 0; e < 4; ++e) u[jj * 4 + e] = nn[e];
-      }
-#pragma unroll
-      for (int cc = 0; cc < CPL; ++cc) dot[cc] = xor_sum<8>(xor_sum<4>(xor_sum<2>(xor_sum<1>(d0[cc] + d1[cc]))));
+    auto step = [&](int t, int t_next) {
+      float un[DR], rr[DR], ww[DR], aa[DR];
+      load(us, t_next, un), load(rs, t, rr), load(ws, t, ww), load(as, t, aa);
+      float o0[CPL], o1[CPL], d0[CPL], d1[CPL];
 #pragma unroll
       for (int cc = 0; cc < CPL; ++cc) {
-        const float o = xor_sum<8>(xor_sum<4>(xor_sum<2>(xor_sum<1>(o0[cc] + o1[cc]))));
+        const float v = vs[t][cg * CPL + cc];
+        o0[cc] = o1[cc] = d0[cc] = d1[cc] = 0.f;
+#pragma unroll
+        for (int e = 0; e < DR; ++e) {
+          float& S = st[cc][e];
+          S = fmaf(ww[e], S, u[e] * fmaf(-aa[e], dot[cc], v));
+          float& o = e & 1 ? o1[cc] : o0[cc];
+          float& d = e & 1 ? d1[cc] : d0[cc];
+          o = fmaf(rr[e], S, o);
+          d = fmaf(un[e], S, d);
+        }
+      }
+#pragma unroll
+      for (int cc = 0; cc < CPL; ++cc) dot[cc] = lanes_sum<LANES>(d0[cc] + d1[cc]);
+#pragma unroll
+      for (int cc = 0; cc < CPL; ++cc) {
+        const float o = lanes_sum<LANES>(o0[cc] + o1[cc]);
         const int c = cb * kGdCols + cg * CPL + cc;
         if (r == 0 && c < Dv) out[(int64_t)(r0 + c0 + t) * ldo + h * Dv + c] = o;
       }
+#pragma unroll
+      for (int e = 0; e < DR; ++e) u[e] = un[e];
+    };
+    if (nt == ROWS) {  // unrolled: the rows' LDS reads run ahead of the walk
+#pragma unroll
+      for (int t = 0; t < ROWS; ++t) step(t, t + 1 < ROWS ? t + 1 : t);
+    } else {
+      for (int t = 0; t < nt; ++t) step(t, min(t + 1, nt - 1));
     }
   }
 #pragma unroll
@@ -432,13 +441,13 @@ extern "C" int mi_diff_heads(const float* o, int64_t ldo_in, const float* lam, i
   return check_launch();
 }
 
-// key channels per lane: the head's channels padded to 64, 128 or 256 over a column's sixteen lanes
-static int gd_dr(int D) { return D <= 64 ? 4 : D <= 128 ? 8 : D <= 256 ? 16 : 0; }
+// a head's key channels as the kernel keeps them: padded to 64, 128 or 256
+static int gd_pad(int D) { return D <= 64 ? 64 : D <= 128 ? 128 : D <= 256 ? 256 : 0; }
 
 extern "C" int64_t mi_general_delta_state_elems(int H, int D, int Dv) {
-  const int dr = gd_dr(D);
-  if (H < 1 || D < 1 || Dv < 1 || !dr) return -1;
-  return (int64_t)H * ((Dv + kGdCols - 1) / kGdCols) * kGdCols * kGdLanes * dr;
+  const int dp = gd_pad(D);
+  if (H < 1 || D < 1 || Dv < 1 || !dp) return -1;
+  return (int64_t)H * ((Dv + kGdCols - 1) / kGdCols) * kGdCols * dp;
 }
 
 extern "C" int mi_general_delta(const float* proj, int64_t ld, int r_off, int k_off, int v_off, int a_off,
@@ -450,16 +459,16 @@ extern "C" int mi_general_delta(const float* proj, int64_t ld, int r_off, int k_
   for (int off : {r_off, k_off, a_off})
     if (off < 0 || ld < off + (int64_t)H * D) return MI_EINVAL;
   if (v_off < 0 || ld < v_off + (int64_t)H * Dv) return MI_EINVAL;
-  const int dr = gd_dr(D), blocks = (Dv + kGdCols - 1) / kGdCols;
-  if (!dr || H > 65535 || blocks > 65535) return MI_EUNSUPPORTED;
+  const int dp = gd_pad(D), blocks = (Dv + kGdCols - 1) / kGdCols;
+  if (!dp || H > 65535 || blocks > 65535) return MI_EUNSUPPORTED;
   if (rows == 0) return MI_OK;
   const dim3 grid(n_seqs, H, blocks);
-#define MI_GD(DR, CPL, ROWS)                                                                                            \
-  hipLaunchKernelGGL((general_delta_kernel<DR, CPL, ROWS>), grid, dim3(kGdLanes * kGdCols / CPL), 0, S(stream), proj, ld,   \
+#define MI_GD(LANES, DR, CPL, ROWS)                                                                                     \
+  hipLaunchKernelGGL((general_delta_kernel<LANES, DR, CPL, ROWS>), grid, dim3(LANES * kGdCols / CPL), 0, S(stream), proj, ld, \
                      r_off, k_off, v_off, a_off, w_decay, ldw, state, cu_q, kv_lens, slot_ids, H, D, Dv, out, ldo)
-  if (dr == 4) MI_GD(4, 2, 16);
-  else if (dr == 8) MI_GD(8, 2, 16);
-  else MI_GD(16, 2, 8);
+  if (dp == 64) MI_GD(16, 4, 1, 16);
+  else if (dp == 128) MI_GD(16, 8, 1, 16);
+  else MI_GD(16, 16, 2, 8);
 #undef MI_GD
   return check_launch();
 }
