@@ -736,7 +736,7 @@ int mi_moe_combine_f32(const float* y, const float* h, int64_t ldh, const int32_
 #define MI_ACT_SOFTCAP   5  /* alpha tanh(z / alpha): the epilogue's alpha is the cap (mi_gemm_any_act, no w2) */
 #define MI_ACT_CLAMPED_GLU 6 /* two weights: g = min(x w^T, limit), u = clamp(x w2^T, -limit, limit);
                               * y = g sigmoid(1.702 g) (u + 1)  (mi_gemm_any_grouped_glu) */
-#define MI_ACT_TANH      7
+#define MI_ACT_TANH      7  /* this and the next: mi_gemm_any_segments only */
 #define MI_ACT_DECAY     8  /* exp(-exp(-1/2) sigmoid(z)): a decay between exp(-exp(-1/2)) and 1 */
 /* mi_gemm_any with an epilogue: v = x w^T + bias (bias may be NULL); w2 != NULL: y = alpha * act(v) * (x w2^T + bias2),
  * else y = alpha * act(v). */

@@ -51,9 +51,9 @@ struct GemmAnyArgs {
   const float* row_scale;
   const int32_t* row_scale_rows;
   float limit;  // MI_ACT_CLAMPED_GLU
-  // act_segments: `act` applies to the features n >= act_from only, `act2` to those from act2_from (>= act_from) on -
+  // extended epilogue: `act` applies to the features n >= act_from only, `act2` to those from act2_from (>= act_from) on -
   // several projections of one input, each with an activation of its own, as one product
-  bool act_segments;
+  bool ext;
   int act_from, act2, act2_from;
 };
 
@@ -72,13 +72,19 @@ __device__ __forceinline__ float act_f(int act, float z) {
     case MI_ACT_GELU_TANH: return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
     case MI_ACT_GELU_ERF: return 0.5f * z * (1.f + erff(z * 0.7071067811865476f));
     case MI_ACT_SIGMOID: return 1.f / (1.f + expf(-z));
-    case MI_ACT_TANH: return tanhf(z);
-    case MI_ACT_DECAY: return expf(-0.6065306597126334f / (1.f + expf(-z)));  // exp(-exp(-1/2) sigmoid(z))
     default: return z;  // (MI_ACT_SOFTCAP is finish()'s: it needs the cap)
   }
 }
-// what every kernel does to an accumulator (pair) before it stores it
-template <bool DUAL>
+// the activations of the extended epilogue
+__device__ __forceinline__ float act_ext_f(int act, float z) {
+  if (act == MI_ACT_TANH) return tanhf(z);
+  if (act == MI_ACT_DECAY) return expf(-0.6065306597126334f / (1.f + expf(-z)));  // exp(-exp(-1/2) sigmoid(z))
+  return act_f(act, z);
+}
+// what every kernel does to an accumulator (pair) before it stores it.  EXT: the epilogue with the activation segments and
+// the activations only they use - kernels of their own, because a longer epilogue costs every tile kernel registers (7 % of
+// a prefill step of models that never take these branches)
+template <bool DUAL, bool EXT>
 __device__ __forceinline__ float finish(const GemmAnyArgs& a, int64_t m, int64_t yrow, int n, float v, float v2) {
   if (a.row_scale) {
     const float rs = a.row_scale[a.row_scale_rows ? a.row_scale_rows[m] : m];
@@ -93,8 +99,8 @@ __device__ __forceinline__ float finish(const GemmAnyArgs& a, int64_t m, int64_t
     } else {
       v = act_f(a.act, v) * v2;
     }
-  } else if (a.act_segments) {
-    if (n >= a.act_from) v = n >= a.act2_from ? act_f(a.act2, v) : act_f(a.act, v);
+  } else if constexpr (EXT) {
+    if (n >= a.act_from) v = n >= a.act2_from ? act_ext_f(a.act2, v) : act_ext_f(a.act, v);
   } else {
     v = a.act == MI_ACT_SOFTCAP ? tanhf(v / a.alpha) : act_f(a.act, v);  // (times alpha below: alpha tanh(v / alpha))
   }
@@ -148,7 +154,7 @@ __device__ __forceinline__ void load8<float>(const float* p, int n_valid, bool v
 // ---------------------------------------------------------------------------------------------------------------
 // exact kernel: 64 x 64 tile, 256 threads, 4 x 4 outputs per thread, k ascending
 // ---------------------------------------------------------------------------------------------------------------
-template <typename TW, bool DUAL, int RT>  // RT rows per thread: a 64 x 64 tile (4) or 16 x 64 (1: few features, many rows)
+template <typename TW, bool DUAL, int RT, bool EXT>  // RT rows per thread: a 64 x 64 tile (4) or 16 x 64 (1: few features, many rows)
 __global__ __launch_bounds__(256) void gemm_any_fma_kernel(GemmAnyArgs a) {
   constexpr int BM = 16 * RT, BN = 64, BK = 32, PAD = 4;
   __shared__ float As[BK][BM + PAD];
@@ -202,7 +208,7 @@ __global__ __launch_bounds__(256) void gemm_any_fma_kernel(GemmAnyArgs a) {
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
       if (n >= a.N) continue;
-      a.y[yrow * a.ldy + n] = finish<DUAL>(a, m, yrow, n, acc[0][i][j], acc[DUAL ? 1 : 0][i][j]);
+      a.y[yrow * a.ldy + n] = finish<DUAL, EXT>(a, m, yrow, n, acc[0][i][j], acc[DUAL ? 1 : 0][i][j]);
     }
   }
 }
@@ -213,7 +219,7 @@ __global__ __launch_bounds__(256) void gemm_any_fma_kernel(GemmAnyArgs a) {
 // K in steps of 64 (a weight row's piece = one 128-byte line).  LDS holds the tile's x rows and weight rows as bf16
 // [64][64 + 8].
 // ---------------------------------------------------------------------------------------------------------------
-template <bool DUAL, int FM, int FN>  // a wave's tile: FM x FN fragments of 16 x 16; the workgroup's: 2 x 2 waves
+template <bool DUAL, int FM, int FN, bool EXT>  // a wave's tile: FM x FN fragments of 16 x 16; the workgroup's: 2 x 2 waves
 __global__ __launch_bounds__(256) void gemm_any_mfma_kernel(GemmAnyArgs a) {
   constexpr int BM = 32 * FM, BN = 32 * FN, BK = 64, LD = BK + 8;
   constexpr int ND = DUAL ? 2 : 1;
@@ -334,7 +340,7 @@ __global__ __launch_bounds__(256) void gemm_any_mfma_kernel(GemmAnyArgs a) {
       float v[4];
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        v[r] = n + r < a.N ? finish<DUAL>(a, m, yrow, n + r, acc[0][i][j][r], acc[ND - 1][i][j][r]) : 0.f;
+        v[r] = n + r < a.N ? finish<DUAL, EXT>(a, m, yrow, n + r, acc[0][i][j][r], acc[ND - 1][i][j][r]) : 0.f;
       float* yp = a.y + yrow * a.ldy + n;
       if (n + 4 <= a.N && (a.ldy % 4 == 0) && dev_aligned16(a.y)) {
         *reinterpret_cast<float4*>(yp) = float4{v[0], v[1], v[2], v[3]};
@@ -353,7 +359,7 @@ __global__ __launch_bounds__(256) void gemm_any_mfma_kernel(GemmAnyArgs a) {
 // 256 contiguous bytes of every weight row per round), operands go from memory straight into MFMA fragments - no LDS
 // staging, no barrier inside the K loop - and the waves' accumulators are added in wave order through LDS at the end.
 // ---------------------------------------------------------------------------------------------------------------
-template <bool DUAL, int MF>  // MF fragments of 16 rows
+template <bool DUAL, int MF, bool EXT>  // MF fragments of 16 rows
 __global__ __launch_bounds__(256) void gemm_any_skinny_kernel(GemmAnyArgs a) {
   __shared__ __attribute__((aligned(16))) float red[3][DUAL ? 2 : 1][MF][64][4];
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
@@ -436,7 +442,7 @@ __global__ __launch_bounds__(256) void gemm_any_skinny_kernel(GemmAnyArgs a) {
     for (int r = 0; r < 4; ++r) {
       const int n = n0 + (lane >> 4) * 4 + r;
       if (n >= a.N) continue;
-      a.y[yrow * a.ldy + n] = finish<DUAL>(a, m, yrow, n, acc[0][f][r], acc[DUAL ? 1 : 0][f][r]);
+      a.y[yrow * a.ldy + n] = finish<DUAL, EXT>(a, m, yrow, n, acc[0][f][r], acc[DUAL ? 1 : 0][f][r]);
     }
   }
 }
@@ -445,7 +451,7 @@ __global__ __launch_bounds__(256) void gemm_any_skinny_kernel(GemmAnyArgs a) {
 // few rows: one wave per output feature and batch of MT rows (blockIdx.y); the lanes take K in pieces of 8, ascending,
 // 16-byte loads where the operands allow it, then a butterfly over the lanes
 // ---------------------------------------------------------------------------------------------------------------
-template <typename TW, int MT, bool DUAL>
+template <typename TW, int MT, bool DUAL, bool EXT>
 __global__ __launch_bounds__(256) void gemm_any_rows_kernel(GemmAnyArgs a) {
   const int lane = threadIdx.x & 63;
   const int n = blockIdx.x * 4 + (threadIdx.x >> 6);
@@ -481,12 +487,12 @@ __global__ __launch_bounds__(256) void gemm_any_rows_kernel(GemmAnyArgs a) {
     const float v2 = DUAL ? wave_sum(acc[DUAL ? 1 : 0][r]) : 0.f;
     if (lane == 0 && xr[r] >= 0) {
       const int64_t yrow = a.y_rows ? a.y_rows[m0 + r] : m0 + r;
-      a.y[yrow * a.ldy + n] = finish<DUAL>(a, m0 + r, yrow, n, v, v2);
+      a.y[yrow * a.ldy + n] = finish<DUAL, EXT>(a, m0 + r, yrow, n, v, v2);
     }
   }
 }
 
-template <typename TW, bool DUAL>
+template <typename TW, bool DUAL, bool EXT>
 static int launch_any(const GemmAnyArgs& a, int groups, int rows_per_group_max, int mode, hipStream_t st) {
   // mode 0: product (MFMA for bf16 weights, the row kernel for few rows); 1: exact (FMA chains / row kernel, x unrounded)
   // few rows (per group): the weight-streaming row kernel.  Also the exact mode up to 64 rows: a router's few output
@@ -495,19 +501,19 @@ static int launch_any(const GemmAnyArgs& a, int groups, int rows_per_group_max, 
   if (few) {
     const int mt = rows_per_group_max <= 1 ? 1 : rows_per_group_max <= 4 ? 4 : 8;
     const dim3 grid((a.N + 3) / 4, (rows_per_group_max + mt - 1) / mt, groups);
-    if (mt == 1) hipLaunchKernelGGL((gemm_any_rows_kernel<TW, 1, DUAL>), grid, dim3(256), 0, st, a);
-    else if (mt == 4) hipLaunchKernelGGL((gemm_any_rows_kernel<TW, 4, DUAL>), grid, dim3(256), 0, st, a);
-    else hipLaunchKernelGGL((gemm_any_rows_kernel<TW, 8, DUAL>), grid, dim3(256), 0, st, a);
+    if (mt == 1) hipLaunchKernelGGL((gemm_any_rows_kernel<TW, 1, DUAL, EXT>), grid, dim3(256), 0, st, a);
+    else if (mt == 4) hipLaunchKernelGGL((gemm_any_rows_kernel<TW, 4, DUAL, EXT>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((gemm_any_rows_kernel<TW, 8, DUAL, EXT>), grid, dim3(256), 0, st, a);
     return check_launch();
   }
   const dim3 grid((a.N + 63) / 64, (rows_per_group_max + 63) / 64, groups);
   if constexpr (sizeof(TW) == 2) {
     if (mode == 0 && rows_per_group_max >= 512 && a.N >= 128) {  // prefill-sized: 128-row tiles, 128 (SwiGLU: 64) features
       if (DUAL) {
-        hipLaunchKernelGGL((gemm_any_mfma_kernel<DUAL, 4, 2>), dim3((a.N + 63) / 64, (rows_per_group_max + 127) / 128, groups),
+        hipLaunchKernelGGL((gemm_any_mfma_kernel<DUAL, 4, 2, EXT>), dim3((a.N + 63) / 64, (rows_per_group_max + 127) / 128, groups),
                            dim3(256), 0, st, a);
       } else {
-        hipLaunchKernelGGL((gemm_any_mfma_kernel<DUAL, 4, 4>), dim3((a.N + 127) / 128, (rows_per_group_max + 127) / 128, groups),
+        hipLaunchKernelGGL((gemm_any_mfma_kernel<DUAL, 4, 4, EXT>), dim3((a.N + 127) / 128, (rows_per_group_max + 127) / 128, groups),
                            dim3(256), 0, st, a);
       }
       return check_launch();
@@ -516,23 +522,23 @@ static int launch_any(const GemmAnyArgs& a, int groups, int rows_per_group_max, 
       // decode-sized: 16-feature workgroups (grouped: tiles of 32 rows, an expert's few rows fill the first)
       if (groups > 1 || rows_per_group_max <= 32) {
         const dim3 g2((a.N + 15) / 16, (rows_per_group_max + 31) / 32, groups);
-        hipLaunchKernelGGL((gemm_any_skinny_kernel<DUAL, 2>), g2, dim3(256), 0, st, a);
+        hipLaunchKernelGGL((gemm_any_skinny_kernel<DUAL, 2, EXT>), g2, dim3(256), 0, st, a);
       } else {
         const dim3 g4((a.N + 15) / 16, 1, groups);
-        hipLaunchKernelGGL((gemm_any_skinny_kernel<DUAL, 4>), g4, dim3(256), 0, st, a);
+        hipLaunchKernelGGL((gemm_any_skinny_kernel<DUAL, 4, EXT>), g4, dim3(256), 0, st, a);
       }
       return check_launch();
     }
     if (mode == 0) {
-      hipLaunchKernelGGL((gemm_any_mfma_kernel<DUAL, 2, 2>), grid, dim3(256), 0, st, a);
+      hipLaunchKernelGGL((gemm_any_mfma_kernel<DUAL, 2, 2, EXT>), grid, dim3(256), 0, st, a);
       return check_launch();
     }
   }
   if (a.N <= 64 && rows_per_group_max >= 1024) {  // a router over a prompt: one column of tiles - short tiles, more of them
-    hipLaunchKernelGGL((gemm_any_fma_kernel<TW, DUAL, 1>), dim3(1, (rows_per_group_max + 15) / 16, groups), dim3(256), 0, st, a);
+    hipLaunchKernelGGL((gemm_any_fma_kernel<TW, DUAL, 1, EXT>), dim3(1, (rows_per_group_max + 15) / 16, groups), dim3(256), 0, st, a);
     return check_launch();
   }
-  hipLaunchKernelGGL((gemm_any_fma_kernel<TW, DUAL, 4>), grid, dim3(256), 0, st, a);
+  hipLaunchKernelGGL((gemm_any_fma_kernel<TW, DUAL, 4, EXT>), grid, dim3(256), 0, st, a);
   return check_launch();
 }
 
@@ -542,16 +548,15 @@ using namespace mi;
 
 static int gemm_any_dispatch(const GemmAnyArgs& a, int w_dtype, int groups, int rows_max, int mode, hipStream_t st) {
   if (a.M == 0 || a.N == 0 || rows_max == 0) return MI_OK;
-  if (w_dtype == MI_DTYPE_BF16)
-    return a.w2 ? launch_any<uint16_t, true>(a, groups, rows_max, mode, st) : launch_any<uint16_t, false>(a, groups, rows_max, mode, st);
-  if (w_dtype == MI_DTYPE_F32)
-    return a.w2 ? launch_any<float, true>(a, groups, rows_max, mode, st) : launch_any<float, false>(a, groups, rows_max, mode, st);
-  return MI_EINVAL;
+  if (w_dtype != MI_DTYPE_BF16 && w_dtype != MI_DTYPE_F32) return MI_EINVAL;
+  const bool bf16 = w_dtype == MI_DTYPE_BF16;
+  if (a.w2) return bf16 ? launch_any<uint16_t, true, false>(a, groups, rows_max, mode, st) : launch_any<float, true, false>(a, groups, rows_max, mode, st);
+  if (a.ext) return bf16 ? launch_any<uint16_t, false, true>(a, groups, rows_max, mode, st) : launch_any<float, false, true>(a, groups, rows_max, mode, st);
+  return bf16 ? launch_any<uint16_t, false, false>(a, groups, rows_max, mode, st) : launch_any<float, false, false>(a, groups, rows_max, mode, st);
 }
 
-static bool act_ok(int act) {
-  return (act >= MI_ACT_NONE && act <= MI_ACT_SOFTCAP) || act == MI_ACT_TANH || act == MI_ACT_DECAY;
-}
+static bool act_ok(int act) { return act >= MI_ACT_NONE && act <= MI_ACT_SOFTCAP; }
+static bool act_ext_ok(int act) { return (act_ok(act) && act != MI_ACT_SOFTCAP) || act == MI_ACT_TANH || act == MI_ACT_DECAY; }
 
 extern "C" int mi_gemm_any(const float* x, int64_t ldx, const void* w, int w_dtype, float* y, int64_t ldy, int M, int N,
                            int K, float alpha, int exact, mi_stream stream) {
@@ -570,8 +575,8 @@ extern "C" int mi_gemm_any_act(const float* x, int64_t ldx, const void* w, const
 extern "C" int mi_gemm_any_segments(const float* x, int64_t ldx, const void* w, int w_dtype, const float* bias, int act,
                                     int act_from, int act2, int act2_from, float* y, int64_t ldy, int M, int N, int K,
                                     int exact, mi_stream stream) {
-  if (!x || !w || !y || M < 0 || N < 0 || K < 1 || ldx < K || ldy < N || !act_ok(act) || !act_ok(act2)) return MI_EINVAL;
-  if (act == MI_ACT_SOFTCAP || act2 == MI_ACT_SOFTCAP || act_from < 0 || act2_from < act_from) return MI_EINVAL;
+  if (!x || !w || !y || M < 0 || N < 0 || K < 1 || ldx < K || ldy < N || !act_ext_ok(act) || !act_ext_ok(act2)) return MI_EINVAL;
+  if (act_from < 0 || act2_from < act_from) return MI_EINVAL;
   GemmAnyArgs a{x, ldx, w, nullptr, y, ldy, M, N, K, 1.0f, nullptr, nullptr, nullptr, bias, nullptr, act, nullptr, 0, 0, 0, 0, nullptr, nullptr, 0.f, true, act_from, act2, act2_from};
   return gemm_any_dispatch(a, w_dtype, 1, M, exact ? 1 : 0, S(stream));
 }

@@ -841,7 +841,7 @@ class GeneralDeltaMixer(nn.Module):
         ctx, m = get_context(), self.proj
         off = {name: o for name, (o, _) in m.offsets.items()}
         y = ops.gemm_any_segments(h, m.weight, m.bias, _C.ACT_SIGMOID, off["a"], _C.ACT_TANH, off["w1"])
-        w = ops.gemm_any_act(m.cols(y, "w1"), self.w2, bias=self.w0, act=_C.ACT_DECAY)
+        w = ops.gemm_any_segments(m.cols(y, "w1"), self.w2, self.w0, _C.ACT_DECAY, 0)
         o = ops.general_delta(y, off["r"], off["k"], off["v"], off["a"], w, self.state[lane], ctx.cu_seqlens_q, ctx.kv_lens,
                               ctx.state_slots, self.H, self.D, self.D)
         ops.head_norm_gate(o, m.cols(y, "g"), _C.ACT_SIGMOID, self.norm, self.H, self.D, self.eps)
