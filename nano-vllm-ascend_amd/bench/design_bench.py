@@ -161,7 +161,7 @@ def munizen_config(s: dict) -> dict:
     W, D, H, G = s["width"], s["dim"], s["heads"], s["kv_heads"]
     att = {"type": "attention",
            "mixer": {"heads": H, "kv_heads": G, "dim": D // 2, "vdim": D, "mask": {"size": s["window"]}, "scale": (D // 2) ** -0.5,
-                     "diff": 0.6, "rot": {"base": 10000.0, "dims": D // 2}}}
+                     "diff": 0.5, "rot": {"base": 10000.0, "dims": D // 2}}}
     rec = {"type": "general_delta", "mixer": {"heads": H, "dim": D, "rank": W // 16}}
     ff = {"kind": "dense", "ff": s["top"] * s["ff"]}
     n = s["layers"]
