@@ -661,6 +661,11 @@ int mi_gemm_any_grouped(const float* x, int64_t ldx, const int32_t* x_rows, cons
 /* out[i] = table[ids[i]] widened to fp32, times scale. */
 int mi_embedding_f32(const int64_t* ids, const void* table, int table_dtype, float* out, int n, int width, int vocab,
                      float scale, mi_stream stream);
+/* The same plus sinusoids of the row's position (cu_q, kv_lens: as in mi_paged_attention_f32): channel 2i gets
+ * sin(pos * inv_freq[i]), channel 2i + 1 cos of the same angle (an fp32 product); inv_freq [(width + 1) / 2]. */
+int mi_embedding_sinusoid_f32(const int64_t* ids, const void* table, int table_dtype, float* out, int n, int width, int vocab,
+                              float scale, const float* inv_freq, const int32_t* cu_q, const int32_t* kv_lens, int n_seqs,
+                              mi_stream stream);
 /* LayerNorm (mean and mean squared deviation in fp32, eps inside the root, weight and bias) of each row of y;
  * add_to_out != 0: out += LN(y) (a residual stream whose norm sits on the sublayer's output). */
 int mi_layernorm_f32(const float* y, int64_t ldy, const float* w, const float* b, float* out, int64_t ldo, int rows,
@@ -736,8 +741,9 @@ int mi_moe_combine_f32(const float* y, const float* h, int64_t ldh, const int32_
 #define MI_ACT_SOFTCAP   5  /* alpha tanh(z / alpha): the epilogue's alpha is the cap (mi_gemm_any_act, no w2) */
 #define MI_ACT_CLAMPED_GLU 6 /* two weights: g = min(x w^T, limit), u = clamp(x w2^T, -limit, limit);
                               * y = g sigmoid(1.702 g) (u + 1)  (mi_gemm_any_grouped_glu) */
-#define MI_ACT_TANH      7  /* this and the next: mi_gemm_any_segments only */
+#define MI_ACT_TANH      7  /* this and MI_ACT_DECAY: mi_gemm_any_segments only */
 #define MI_ACT_DECAY     8  /* exp(-exp(-1/2) sigmoid(z)): a decay between exp(-exp(-1/2)) and 1 */
+#define MI_ACT_RELU2     9  /* max(z, 0)^2 (everywhere) */
 /* mi_gemm_any with an epilogue: v = x w^T + bias (bias may be NULL); w2 != NULL: y = alpha * act(v) * (x w2^T + bias2),
  * else y = alpha * act(v). */
 int mi_gemm_any_act(const float* x, int64_t ldx, const void* w, const void* w2, int w_dtype, const float* bias,
@@ -786,11 +792,12 @@ int mi_paged_attention_f32(const float* q, int64_t ldq, const void* k_cache, con
  * heads than key heads (a token's value heads side by side in one row, v_cache possibly pointing at a column of it) every
  * query head weighs the values of several key/value heads at once: out [rows][H][Dv] with Dv the width read.  The same
  * with narrow value heads lets several key heads SHARE a value head (maps of one head over the same values).
- * chunk > 0: position i sees only the keys of its own chunk, floor(i / chunk) = floor(j / chunk), on top of the window. */
+ * chunk > 0: position i sees only the keys of its own chunk, floor(i / chunk) = floor(j / chunk), on top of the window.
+ * kept > 0: the first `kept` keys of a sequence stay visible (j < kept, j <= i) whatever window and chunk say. */
 int mi_paged_attention_ext(const float* q, int64_t ldq, const void* k_cache, const void* v_cache, int64_t ldv,
                            int cache_dtype, const int32_t* block_tables, int table_cols, const int32_t* cu_q,
                            const int32_t* kv_lens, int n_seqs, int rows, int H, int G, int D, int Dv, int block_size,
-                           int window, int chunk, float scale, int bias_kind, const float* bias_p1, const float* bias_p2,
+                           int window, int chunk, int kept, float scale, int bias_kind, const float* bias_p1, const float* bias_p2,
                            const float* sink, float softcap, int value_heads, const float* gate, int64_t ldg, float* out,
                            int64_t ldo, float* workspace, int64_t workspace_elems, mi_stream stream);
 /* res += mult * y (y may be NULL); w != NULL: out = res / sqrt(mean(res^2) + eps) * (w + shift) per row. */
@@ -826,11 +833,11 @@ int mi_latent_prepare(const float* proj, int64_t ld, const float* q, int64_t ldq
                       const float* inv_freq, const float* norm_w, float eps, const int32_t* cu_q, const int32_t* kv_lens,
                       int n_seqs, void* cache, int cache_dtype, const int32_t* slots, float* qx, int64_t ldqx, int rows,
                       mi_stream stream);
-/* ids = the top_k largest logits (descending; equal: lower index), weights = softmax over those.  n_outputs <= 512. */
-int mi_route_topk(const float* logits, int64_t ld, int n_tokens, int n_outputs, int top_k, int32_t* ids, float* weights,
-                  mi_stream stream);
-/* out[t] = sum_k weights[t][k] * y[t * top_k + k] + sigmoid(shared_gate[t]) * shared[t] (shared may be NULL; weights may be
- * NULL: every weight 1). */
+/* ids = the top_k largest logits (descending; equal: lower index), weights = scale * softmax over those.  n_outputs <= 512. */
+int mi_route_topk(const float* logits, int64_t ld, int n_tokens, int n_outputs, int top_k, float scale, int32_t* ids,
+                  float* weights, mi_stream stream);
+/* out[t] = sum_k weights[t][k] * y[t * top_k + k] + sigmoid(shared_gate[t]) * shared[t] (shared may be NULL; shared_gate
+ * may be NULL: the shared part as it is; weights may be NULL: every weight 1). */
 int mi_moe_combine_shared(const float* y, const int32_t* ids, const float* weights, int n_tokens, int top_k, int width,
                           const float* shared, int64_t ld_shared, const float* shared_gate, int64_t ld_gate, float* out,
                           int64_t ldo, mi_stream stream);
@@ -841,6 +848,12 @@ int mi_moe_combine_shared(const float* y, const int32_t* ids, const float* weigh
 int mi_gated_norm_add_f32(float* res, int64_t ldr, const float* y, int64_t ldy, const float* gate_pre, int64_t ldg,
                           const float* w_post, float eps, const float* w_next, float* out, int64_t ldo, int rows, int width,
                           mi_stream stream);
+/* The same without a gate for an output still in parts: v = sum_k weights[row][k] * y[row * parts + k] + shared[row]
+ * (y [rows * parts][width]; weights may be NULL: ones; shared may be NULL), res += v / sqrt(mean(v^2) + eps) * w_post;
+ * w_next != NULL: out = res / sqrt(mean(res^2) + eps) * w_next. */
+int mi_parts_norm_add_f32(float* res, int64_t ldr, const float* y, int parts, const float* weights, const float* shared,
+                          int64_t ld_shared, const float* w_post, float eps, const float* w_next, float* out, int64_t ldo,
+                          int rows, int width, mi_stream stream);
 #define MI_DECAY_HEAD   0  /* a_t = decay[h]: one constant per head */
 #define MI_DECAY_FORGET 1  /* a_t = f_t = lower + (1 - lower) sigmoid(z_t + f_bias) per key channel; k_t = 1 - f_t */
 /* Floats of state one sequence slot holds for mi_linear_attention (the kernel's own thread-order layout), or -1 when D
@@ -864,11 +877,13 @@ int mi_linear_attention(const float* proj, int64_t ld, int q_off, int k_off, int
  * or (i, i + rot_dims/2): */
 #define MI_ROT_INTERLEAVED 0
 #define MI_ROT_HALVES      1
-/* unit_norm: then every head is divided by sqrt(mean(head^2) + eps); key heads times k_mult on top.  k_cache != NULL: the
+/* unit_norm: then every head is divided by sqrt(mean(head^2) + eps) and multiplied by q_norm / k_norm [D] (the same for every
+ * head; NULL: ones); key heads times k_mult on top.  k_cache != NULL: the
  * key heads go to the paged cache [blocks][G][block_size][D] instead of back in place; v_cache != NULL: the row's Gv value
  * heads [Dv] at v_off are copied to [blocks][Gv][block_size][Dv]; slots [rows] (< 0: the row stores nothing). */
 int mi_rotary_store(float* proj, int64_t ld, int q_off, int k_off, int v_off, int H, int G, int D, int Gv, int Dv,
-                    int rot_dims, int layout, const float* inv_freq, float amp, int unit_norm, float eps, float k_mult,
+                    int rot_dims, int layout, const float* inv_freq, float amp, int unit_norm, const float* q_norm,
+                    const float* k_norm, float eps, float k_mult,
                     const int32_t* cu_q, const int32_t* kv_lens, int n_seqs, void* k_cache, void* v_cache, int cache_dtype,
                     const int32_t* slots, int rows, int block_size, mi_stream stream);
 /* Mixing of the heads' softmax weights p'_h = sum_g talk[h][g] p_g, applied to read-outs: o [rows][H][n_chunk * Dv] holds

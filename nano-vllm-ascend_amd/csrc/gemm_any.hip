@@ -72,6 +72,7 @@ __device__ __forceinline__ float act_f(int act, float z) {
     case MI_ACT_GELU_TANH: return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
     case MI_ACT_GELU_ERF: return 0.5f * z * (1.f + erff(z * 0.7071067811865476f));
     case MI_ACT_SIGMOID: return 1.f / (1.f + expf(-z));
+    case MI_ACT_RELU2: return fmaxf(z, 0.f) * fmaxf(z, 0.f);
     default: return z;  // (MI_ACT_SOFTCAP is finish()'s: it needs the cap)
   }
 }
@@ -555,7 +556,7 @@ static int gemm_any_dispatch(const GemmAnyArgs& a, int w_dtype, int groups, int 
   return bf16 ? launch_any<uint16_t, false, false>(a, groups, rows_max, mode, st) : launch_any<float, false, false>(a, groups, rows_max, mode, st);
 }
 
-static bool act_ok(int act) { return act >= MI_ACT_NONE && act <= MI_ACT_SOFTCAP; }
+static bool act_ok(int act) { return (act >= MI_ACT_NONE && act <= MI_ACT_SOFTCAP) || act == MI_ACT_RELU2; }
 static bool act_ext_ok(int act) { return (act_ok(act) && act != MI_ACT_SOFTCAP) || act == MI_ACT_TANH || act == MI_ACT_DECAY; }
 
 extern "C" int mi_gemm_any(const float* x, int64_t ldx, const void* w, int w_dtype, float* y, int64_t ldy, int M, int N,

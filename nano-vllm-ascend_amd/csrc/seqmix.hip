@@ -1,6 +1,7 @@
 // Sequence mixers and row operators of the model families that keep their residual stream in 32-bit floats:
 //
 //   mi_embedding_f32            table rows (bf16 or fp32) -> fp32 residual rows
+//   mi_embedding_sinusoid_f32   the same plus sinusoids of the row's position
 //   mi_layernorm_f32            LayerNorm with weight and bias; optionally ADDED to a residual in place
 //                               (x <- x + LN(y): the norm sits on the sublayer's output)
 //   mi_swa_prepare              sliding-window attention, K/V side: ONE root-mean-square norm over a token's whole q
@@ -23,6 +24,7 @@
 //   mi_moe_combine_f32          out[t] = sum_k w[t][k] * (identity expert ? h[t] : y[t * top_k + k])
 //   mi_causal_conv              the convolution with its activation and a "beside the identity" flag (y = x + conv(x))
 //   mi_gated_norm_add_f32       res += rms(y * sigmoid(gate)) * w, and the norm of the sum for the next sublayer
+//   mi_parts_norm_add_f32       the same for an ungated output still in parts (experts' outputs with their weights)
 //   mi_linear_attention         S <- diag(a_t) S + k_t v_t^T, o_t = S^T q_t with a decay per head or a forget gate per
 //                               key channel that also writes (k = 1 - f); read-out norm per head or over all heads, gate
 //   (further down: the pre-norm families' residual stack, minimal gated recurrence, latent and log-biased attention,
@@ -45,6 +47,30 @@ __global__ __launch_bounds__(256) void embedding_f32_kernel(const int64_t* __res
   if (id < 0 || id >= vocab) return;
   for (int c = threadIdx.x; c < width; c += 256)
     out[(int64_t)blockIdx.x * width + c] = ld_f<TT>(table + id * width + c) * scale;
+}
+
+// table row * scale + sinusoids of the row's position: channel 2i gets sin(pos * inv_freq[i]), channel 2i + 1 cos of the same
+// (angle: one fp32 product).  A thread per channel pair.
+template <typename TT>
+__global__ __launch_bounds__(256) void embedding_sinusoid_f32_kernel(const int64_t* __restrict__ ids,
+                                                                     const TT* __restrict__ table, float* __restrict__ out,
+                                                                     int width, int vocab, float scale,
+                                                                     const float* __restrict__ inv_freq,
+                                                                     const int32_t* __restrict__ cu_q,
+                                                                     const int32_t* __restrict__ kv_lens, int n_seqs) {
+  const int row = blockIdx.x;
+  const int64_t id = ids[row];
+  if (id < 0 || id >= vocab) return;
+  const int s = seq_of_row(cu_q, n_seqs, row);
+  const float pos = (float)(kv_lens[s] - (cu_q[s + 1] - cu_q[s]) + (row - cu_q[s]));
+  const TT* src = table + id * width;
+  float* o = out + (int64_t)row * width;
+  for (int i = threadIdx.x; 2 * i < width; i += 256) {
+    float sn, cs;
+    sincosf(pos * inv_freq[i], &sn, &cs);
+    o[2 * i] = fmaf(ld_f<TT>(src + 2 * i), scale, sn);
+    if (2 * i + 1 < width) o[2 * i + 1] = fmaf(ld_f<TT>(src + 2 * i + 1), scale, cs);
+  }
 }
 
 // one workgroup per row; mean, then the mean of squared deviations (two passes over the row, which stays in L1)
@@ -125,6 +151,7 @@ __global__ __launch_bounds__(256) void swa_prepare_kernel(float* __restrict__ pr
 // afterwards needs.
 // chunk > 0: position i sees the keys of its own chunk only (floor(i / chunk) = floor(j / chunk), positions counted from
 // the sequence's start); with the window: both hold.
+// kept > 0: the first `kept` keys of a sequence stay visible from everywhere behind them, whatever window and chunk say.
 struct AttnBias {
   int kind;
   const float* p1;
@@ -133,6 +160,7 @@ struct AttnBias {
   float softcap;
   int value_heads;
   int chunk;
+  int kept;
 };
 // the oldest key position `pos` sees
 __device__ __forceinline__ int first_key(const AttnBias& bias, int pos, int window) {
@@ -140,6 +168,13 @@ __device__ __forceinline__ int first_key(const AttnBias& bias, int pos, int wind
   if (bias.chunk > 0) lo = max(lo, pos - pos % bias.chunk);
   return lo;
 }
+// Kept keys lie away from the window: a walk over the keys counts u from lo - min(kept, lo) on, the u below lo stand for
+// the kept keys that are older than lo (gap = lo - min(kept, lo) further down), the others for themselves - one run of
+// numbers without holes, so that kept and window keys share the rounds of 32 / 64.  lo: the oldest key of the walk's first
+// row by window and chunk.
+__device__ __forceinline__ int kept_gap(const AttnBias& bias, int lo) { return lo - min(bias.kept, lo); }
+template <bool KEEP>
+__device__ __forceinline__ int key_at(int u, int lo, int gap) { return KEEP && u < lo ? u - gap : u; }
 __device__ __forceinline__ float capped(const AttnBias& bias, float s) {
   return bias.softcap > 0.f ? bias.softcap * tanhf(s / bias.softcap) : s;
 }
@@ -205,8 +240,9 @@ __global__ __launch_bounds__(256) void swa_attention_kernel(const float* __restr
 #pragma unroll
   for (int i = 0; i < VPL; ++i) acc[i] = 0.f;
   __builtin_amdgcn_wave_barrier();
-  for (int j0 = lo; j0 <= pos; j0 += 64) {
-    const int j = j0 + lane;
+  const int gap = kept_gap(bias, lo);
+  for (int j0 = gap; j0 <= pos; j0 += 64) {
+    const int j = key_at<true>(j0 + lane, lo, gap);
     float sc = -INFINITY;
     if (j <= pos) {
       const int64_t blk = table[j / block_size];
@@ -226,7 +262,7 @@ __global__ __launch_bounds__(256) void swa_attention_kernel(const float* __restr
 #pragma unroll
     for (int i = 0; i < VPL; ++i) acc[i] *= corr;
     for (int jj = 0; jj < n_keys; ++jj) {
-      const int jk = j0 + jj;
+      const int jk = key_at<true>(j0 + jj, lo, gap);
       const int64_t blk = table[jk / block_size];
       const TC* vr = v_cache + ((blk * Gv + gv) * block_size + jk % block_size) * ldv;
       const float pj = ps[jj];
@@ -320,8 +356,9 @@ __global__ __launch_bounds__(256) void swa_attention_vec_kernel(const float* __r
 #pragma unroll
       for (int e = 0; e < VEC; ++e) acc[r][e] = 0.f;
     }
-    for (int j0 = lo + 64 * cw; j0 <= hi; j0 += 64 * SPLIT) {
-      const int j = j0 + lane;
+    const int gap = kept_gap(bias, lo);
+    for (int j0 = gap + 64 * cw; j0 <= hi; j0 += 64 * SPLIT) {
+      const int j = key_at<true>(j0 + lane, lo, gap);
       float dots[RPW];
 #pragma unroll
       for (int r = 0; r < RPW; ++r) dots[r] = 0.f;
@@ -346,7 +383,7 @@ __global__ __launch_bounds__(256) void swa_attention_vec_kernel(const float* __r
 #pragma unroll
       for (int r = 0; r < RPW; ++r) {
         const int pos = pos0 + r;
-        const bool vis = r < nr && j <= pos && j >= row_lo[r];
+        const bool vis = r < nr && j <= pos && (j >= row_lo[r] || j < bias.kept);
         const float sc = vis ? capped(bias, dots[r] * scale - dist_bias(hb, pos - j)) : -INFINITY;
         const float m_new = fmaxf(m[r], wave_max(sc));
         const float p = vis ? expf(sc - m_new) : 0.f;
@@ -361,7 +398,7 @@ __global__ __launch_bounds__(256) void swa_attention_vec_kernel(const float* __r
       const int nk = min(64, hi - j0 + 1);
       if (cg * VEC < Dv) {
         for (int jj = kg; jj < nk; jj += kpp) {
-          const int jk = j0 + jj;
+          const int jk = key_at<true>(j0 + jj, lo, gap);
           const int64_t blk = table[jk / block_size];
           float vv[VEC];
           ld_vec<TC, VEC>(v_cache + ((blk * Gv + gv) * block_size + jk % block_size) * ldv + cg * VEC, vv);
@@ -431,7 +468,7 @@ __global__ __launch_bounds__(256) void swa_attention_vec_kernel(const float* __r
 // operand gathers its eight keys' elements.  Scores and weights stay fp32 quantities: q and p enter the MFMAs as
 // bf16 hi + lo pairs (two MFMAs each, products exact, fp32 accumulation: 16 mantissa bits of q and p against the 8 of a
 // plain bf16 operand), scale, distance bias, mask, running maximum and sum are fp32 VALU work on the accumulators.
-template <int DKM, int DVM, bool PAIR>
+template <int DKM, int DVM, bool PAIR, bool KEEP>  // KEEP: bias.kept > 0
 __global__ __launch_bounds__(256) void swa_attention_mfma_kernel(const float* __restrict__ q, int64_t ldq,
                                                                  const uint16_t* __restrict__ k_cache,
                                                                  const uint16_t* __restrict__ v_cache,
@@ -481,19 +518,20 @@ __global__ __launch_bounds__(256) void swa_attention_mfma_kernel(const float* __
       ql[ks] = as_frag(u32x4{pack_bf(lo[0], lo[1]), pack_bf(lo[2], lo[3]), pack_bf(lo[4], lo[5]), pack_bf(lo[6], lo[7])});
     }
     const int lo_key = first_key(bias, pos0, window), hi_key = pos0 + nr - 1;
+    const int gap = KEEP ? kept_gap(bias, lo_key) : lo_key;
     const int my_pos = pos0 + qi;
     const int my_lo = first_key(bias, my_pos, window);
     float m = -INFINITY, l = 0.f;
     f32x4 oacc[DVM];
 #pragma unroll
     for (int dt = 0; dt < DVM; ++dt) oacc[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int j0 = lo_key; j0 <= hi_key; j0 += 32) {
+    for (int j0 = gap; j0 <= hi_key; j0 += 32) {
       f32x4 sacc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
       for (int t = 0; t < 2; ++t) {
         // this lane's row of the K operand; rows beyond the last key repeat it (their scores are masked below), so
         // that every load is unconditional and a round's loads are all in flight together
-        const int key = min(j0 + t * 16 + qi, hi_key);
+        const int key = key_at<KEEP>(min(j0 + t * 16 + qi, hi_key), lo_key, gap);
         const uint16_t* kr =
             k_cache + (int64_t)cache_row(table, key, G, g, block_size, bs_shift) * D + kg * 8;
 #pragma unroll
@@ -511,8 +549,8 @@ __global__ __launch_bounds__(256) void swa_attention_mfma_kernel(const float* __
       float mx = -INFINITY;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
-        const int key = j0 + (e >> 2) * 16 + kg * 4 + (e & 3);
-        vis[e] = qi < nr && key <= my_pos && key >= my_lo;
+        const int key = key_at<KEEP>(j0 + (e >> 2) * 16 + kg * 4 + (e & 3), lo_key, gap);
+        vis[e] = qi < nr && key <= my_pos && (key >= my_lo || (KEEP && key < bias.kept));
         sc[e] = sacc[e >> 2][e & 3] * scale;
         dist[e] = my_pos - key;
       }
@@ -557,7 +595,8 @@ __global__ __launch_bounds__(256) void swa_attention_mfma_kernel(const float* __
       const uint16_t* vrow[8];
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
-        const int key = min(j0 + (e >> 2) * 16 + kg * 4 + (e & 3), hi_key);  // (beyond the last key: weight 0)
+        // (beyond the last key: weight 0)
+        const int key = key_at<KEEP>(min(j0 + (e >> 2) * 16 + kg * 4 + (e & 3), hi_key), lo_key, gap);
         vrow[e] = v_cache + (int64_t)cache_row(table, key, Gv, gv, block_size, bs_shift) * (int)ldv +
                   (PAIR ? 2 * qi : qi);
       }
@@ -622,7 +661,7 @@ __global__ __launch_bounds__(256) void swa_attention_mfma_kernel(const float* __
 // consecutive rows of one head, so every K and V element the workgroup loads serves all of the group's heads (latent
 // attention: ONE cache row for every head).  Its four waves take the rounds of 32 keys in turn and merge their (max, sum,
 // accumulator) triples through LDS.  Arithmetic as in the prompt form: q and the softmax weights as bf16 hi + lo pairs.
-template <int DKM, int DVM, bool PAIR>
+template <int DKM, int DVM, bool PAIR, bool KEEP>
 __global__ __launch_bounds__(256) void paged_attention_heads_mfma_kernel(
     const float* __restrict__ q, int64_t ldq, const uint16_t* __restrict__ k_cache, const uint16_t* __restrict__ v_cache,
     const int32_t* __restrict__ block_tables, int table_cols, const int32_t* __restrict__ kv_lens, int H, int G, int D,
@@ -665,11 +704,12 @@ __global__ __launch_bounds__(256) void paged_attention_heads_mfma_kernel(
     ql[ks] = as_frag(u32x4{pack_bf(lo[0], lo[1]), pack_bf(lo[2], lo[3]), pack_bf(lo[4], lo[5]), pack_bf(lo[6], lo[7])});
   }
   const int lo_key = first_key(bias, pos, window), hi_key = pos;
+  const int gap = KEEP ? kept_gap(bias, lo_key) : lo_key;
   float m = -INFINITY, l = 0.f;
   f32x4 oacc[DVM];
 #pragma unroll
   for (int dt = 0; dt < DVM; ++dt) oacc[dt] = f32x4{0.f, 0.f, 0.f, 0.f};
-  for (int j0 = lo_key + 32 * (split * 4 + wave); j0 <= hi_key; j0 += 32 * 4 * n_split) {
+  for (int j0 = gap + 32 * (split * 4 + wave); j0 <= hi_key; j0 += 32 * 4 * n_split) {
     f32x4 sacc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
     // the round's V words are requested together with its K rows (their addresses do not depend on the scores): one
     // memory latency per round instead of two behind one another.  The V^T operand: the lane's eight keys (its
@@ -677,7 +717,8 @@ __global__ __launch_bounds__(256) void paged_attention_heads_mfma_kernel(
     const uint16_t* vrow[8];
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
-      const int key = min(j0 + (e >> 2) * 16 + kg * 4 + (e & 3), hi_key);  // (beyond the last key: weight 0)
+      // (beyond the last key: weight 0)
+      const int key = key_at<KEEP>(min(j0 + (e >> 2) * 16 + kg * 4 + (e & 3), hi_key), lo_key, gap);
       vrow[e] = v_cache + (int64_t)cache_row(table, key, Gv, gv, block_size, bs_shift) * (int)ldv +
                 (PAIR ? 2 * qi : qi);
     }
@@ -694,7 +735,7 @@ __global__ __launch_bounds__(256) void paged_attention_heads_mfma_kernel(
     for (int t = 0; t < 2; ++t) {
       // this lane's row of the K operand; rows beyond the last key repeat it (their scores are masked below), so
       // that every load is unconditional and a round's loads are all in flight together
-      const int key = min(j0 + t * 16 + qi, hi_key);
+      const int key = key_at<KEEP>(min(j0 + t * 16 + qi, hi_key), lo_key, gap);
       const uint16_t* kr =
           k_cache + (int64_t)cache_row(table, key, G, g, block_size, bs_shift) * D + kg * 8;
 #pragma unroll
@@ -712,7 +753,7 @@ __global__ __launch_bounds__(256) void paged_attention_heads_mfma_kernel(
     float mx = -INFINITY;
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
-      const int key = j0 + (e >> 2) * 16 + kg * 4 + (e & 3);
+      const int key = key_at<KEEP>(j0 + (e >> 2) * 16 + kg * 4 + (e & 3), lo_key, gap);
       vis[e] = qi < nh && key <= hi_key;
       sc[e] = sacc[e >> 2][e & 3] * scale;
       dist[e] = pos - key;
@@ -1558,10 +1599,12 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const float* __rest
 }
 
 // ---------------------------------------------------------------------------------------------------------------
-// plain top-k router: the top_k largest logits (equal values: the lower index), weights = softmax over the chosen
+// plain top-k router: the top_k largest logits (equal values: the lower index), weights = scale * softmax over the chosen
+// (= the chosen entries of the softmax over all outputs, divided by their sum)
 // ---------------------------------------------------------------------------------------------------------------
 __global__ __launch_bounds__(256) void route_topk_kernel(const float* __restrict__ logits, int64_t ld, int T, int n,
-                                                         int top_k, int32_t* __restrict__ ids, float* __restrict__ wts) {
+                                                         int top_k, float scale, int32_t* __restrict__ ids,
+                                                         float* __restrict__ wts) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int t = blockIdx.x * 4 + wave;
   if (t >= T) return;
@@ -1603,18 +1646,18 @@ __global__ __launch_bounds__(256) void route_topk_kernel(const float* __restrict
   }
 #pragma unroll
   for (int i = 0; i < EPL; ++i)
-    if (i < n_mine) wts[(int64_t)t * top_k + my_slot[i]] = mine[i] / sum;
+    if (i < n_mine) wts[(int64_t)t * top_k + my_slot[i]] = mine[i] / sum * scale;
 }
 
 // out[t] = sum_k w[t][k] y[t * top_k + k] + sigmoid(shared_gate[t]) * shared[t]   (shared == nullptr: no shared part;
-// wts == nullptr: every weight 1 - experts whose weight already went into their input)
+// shared_gate == nullptr: the shared part as it is; wts == nullptr: every weight 1 - experts whose weight already went into their input)
 __global__ __launch_bounds__(256) void moe_combine_shared_kernel(const float* __restrict__ y, const int32_t* __restrict__ ids,
                                                                  const float* __restrict__ wts, int top_k, int width,
                                                                  const float* __restrict__ shared, int64_t lds_,
                                                                  const float* __restrict__ shared_gate, int64_t ldsg,
                                                                  float* __restrict__ out, int64_t ldo) {
   const int t = blockIdx.x;
-  const float sgate = shared ? sigmoid_f(shared_gate[(int64_t)t * ldsg]) : 0.f;
+  const float sgate = shared_gate ? sigmoid_f(shared_gate[(int64_t)t * ldsg]) : 1.f;
   for (int c = threadIdx.x; c < width; c += 256) {
     float acc = 0.f;
     for (int k = 0; k < top_k; ++k)
@@ -1671,6 +1714,80 @@ __global__ __launch_bounds__(256) void gated_norm_add_f32_kernel(float* __restri
   float* o = out + (int64_t)blockIdx.x * ldo;
   i = 0;
   for (int c = threadIdx.x; c < width; c += 256, ++i) o[c] = (i < KEEP ? kept[i] : r[c]) * rstd2 * w_next[c];
+}
+
+// The same without a gate, for a sublayer output that is still in parts: v = sum_k wts[row][k] y[row * parts + k] +
+// shared[row] (wts == nullptr: weights 1; shared may be nullptr) - a plain output is one part, a sparse feed-forward's the
+// chosen experts' and the shared expert's - then res += v / sqrt(mean(v^2) + eps) * w_post and the next sublayer's norm.
+// One workgroup per row, VEC channels per load; a thread keeps its first KEEP pieces in registers between the passes (VEC 4:
+// rows up to 4096 wide; wider ones are summed again).
+template <int VEC>
+__global__ __launch_bounds__(256) void parts_norm_add_f32_kernel(float* __restrict__ res, int64_t ldr,
+                                                                 const float* __restrict__ y, int parts,
+                                                                 const float* __restrict__ wts,
+                                                                 const float* __restrict__ shared, int64_t lds_,
+                                                                 const float* __restrict__ w_post, float eps,
+                                                                 const float* __restrict__ w_next,
+                                                                 float* __restrict__ out, int64_t ldo, int width) {
+  typedef float vec __attribute__((ext_vector_type(VEC)));
+  __shared__ float red[4];
+  constexpr int KEEP = 4, STEP = 256 * VEC;
+  const int64_t row = blockIdx.x;
+  float* r = res + row * ldr;
+  const float* yr = y + row * parts * width;
+  const float* sr = shared ? shared + row * lds_ : nullptr;
+  const float* wr = wts ? wts + row * parts : nullptr;
+  auto at = [](const float* p) { return *reinterpret_cast<const vec*>(p); };
+  auto total = [&](int c) {
+    vec v = (vec)(0.f);
+    for (int k = 0; k < parts; ++k) {
+      const vec p = at(yr + (int64_t)k * width + c);
+      v = wr ? v + p * wr[k] : v + p;
+    }
+    return sr ? v + at(sr + c) : v;
+  };
+  auto square = [](vec v) {
+    float s = 0.f;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) s = fmaf(((const float*)&v)[e], ((const float*)&v)[e], s);
+    return s;
+  };
+  const int c0 = threadIdx.x * VEC;
+  vec kept[KEEP];
+  float sq = 0.f;
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i)
+    if (c0 + i * STEP < width) {
+      kept[i] = total(c0 + i * STEP);
+      sq += square(kept[i]);
+    }
+  for (int c = c0 + KEEP * STEP; c < width; c += STEP) sq += square(total(c));
+  const float rstd = 1.f / sqrtf(block_sum256(sq, red) / (float)width + eps);
+  float sq2 = 0.f;
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i) {
+    const int c = c0 + i * STEP;
+    if (c < width) {
+      kept[i] = at(r + c) + kept[i] * rstd * at(w_post + c);
+      *reinterpret_cast<vec*>(r + c) = kept[i];
+      sq2 += square(kept[i]);
+    }
+  }
+  for (int c = c0 + KEEP * STEP; c < width; c += STEP) {
+    const vec x = at(r + c) + total(c) * rstd * at(w_post + c);
+    *reinterpret_cast<vec*>(r + c) = x;
+    sq2 += square(x);
+  }
+  if (!w_next) return;
+  const float rstd2 = 1.f / sqrtf(block_sum256(sq2, red) / (float)width + eps);
+  float* o = out + row * ldo;
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i) {
+    const int c = c0 + i * STEP;
+    if (c < width) *reinterpret_cast<vec*>(o + c) = kept[i] * rstd2 * at(w_next + c);
+  }
+  for (int c = c0 + KEEP * STEP; c < width; c += STEP)  // (a thread re-reads its own writes)
+    *reinterpret_cast<vec*>(o + c) = at(r + c) * rstd2 * at(w_next + c);
 }
 
 // ---------------------------------------------------------------------------------------------------------------
@@ -1815,7 +1932,8 @@ __global__ __launch_bounds__(256) void row_norm_gate_kernel(float* __restrict__ 
 // One workgroup per step row, a wave per head in turn (H query heads at q_off, G key heads at k_off of the row).  The
 // first rot_dims channels of a head are rotated by the angles pos * inv_freq[i] (fp32 product, sincosf), cos and sin
 // times `amp`: channel pairs (2i, 2i + 1) (layout MI_ROT_INTERLEAVED) or (i, i + rot_dims / 2) (MI_ROT_HALVES).  Then,
-// unit_norm: the head is divided by sqrt(mean(head^2) + eps); key heads are multiplied by k_mult on top.  Query heads
+// unit_norm: the head is divided by sqrt(mean(head^2) + eps) and multiplied by q_norm / k_norm [D] (nullptr: ones; the same
+// for every head); key heads are multiplied by k_mult on top.  Query heads
 // are written back in place.  Key heads go to the paged cache [blocks][G][block_size][D] when k_cache != nullptr (rows
 // with slot < 0 store nothing), else back in place.  v_cache != nullptr: the row's Gv value heads of Dv channels at v_off
 // are copied to [blocks][Gv][block_size][Dv] as they are.
@@ -1823,7 +1941,8 @@ template <typename TC>
 __global__ __launch_bounds__(256) void rotary_store_kernel(float* __restrict__ proj, int64_t ld, int q_off, int k_off,
                                                            int v_off, int H, int G, int D, int Gv, int Dv, int rot_dims,
                                                            int layout, const float* __restrict__ inv_freq, float amp,
-                                                           int unit_norm, float eps, float k_mult,
+                                                           int unit_norm, const float* __restrict__ q_norm,
+                                                           const float* __restrict__ k_norm, float eps, float k_mult,
                                                            const int32_t* __restrict__ cu_q,
                                                            const int32_t* __restrict__ kv_lens, int n_seqs,
                                                            TC* __restrict__ k_cache, TC* __restrict__ v_cache,
@@ -1858,6 +1977,11 @@ __global__ __launch_bounds__(256) void rotary_store_kernel(float* __restrict__ p
       float sq = 0.f;
       for (int d = lane; d < D; d += 64) sq = fmaf(hv[d], hv[d], sq);
       mult *= 1.f / sqrtf(wave_sum(sq) / (float)D + eps);
+      const float* nw = is_k ? k_norm : q_norm;
+      if (nw) {
+        for (int d = lane; d < D; d += 64) hv[d] *= nw[d];
+        __builtin_amdgcn_wave_barrier();
+      }
     }
     if (is_k && k_cache) {
       if (slot >= 0) {
@@ -1916,6 +2040,21 @@ extern "C" int mi_embedding_f32(const int64_t* ids, const void* table, int table
   return check_launch();
 }
 
+extern "C" int mi_embedding_sinusoid_f32(const int64_t* ids, const void* table, int table_dtype, float* out, int n, int width,
+                                         int vocab, float scale, const float* inv_freq, const int32_t* cu_q,
+                                         const int32_t* kv_lens, int n_seqs, mi_stream stream) {
+  if (!ids || !table || !out || !inv_freq || !cu_q || !kv_lens || n < 0 || width < 1 || n_seqs < 1) return MI_EINVAL;
+  if (n == 0) return MI_OK;
+  if (table_dtype == MI_DTYPE_BF16)
+    hipLaunchKernelGGL((embedding_sinusoid_f32_kernel<uint16_t>), dim3(n), dim3(256), 0, S(stream), ids,
+                       static_cast<const uint16_t*>(table), out, width, vocab, scale, inv_freq, cu_q, kv_lens, n_seqs);
+  else if (table_dtype == MI_DTYPE_F32)
+    hipLaunchKernelGGL((embedding_sinusoid_f32_kernel<float>), dim3(n), dim3(256), 0, S(stream), ids,
+                       static_cast<const float*>(table), out, width, vocab, scale, inv_freq, cu_q, kv_lens, n_seqs);
+  else return MI_EINVAL;
+  return check_launch();
+}
+
 extern "C" int mi_layernorm_f32(const float* y, int64_t ldy, const float* w, const float* b, float* out, int64_t ldo,
                                 int rows, int width, float eps, int add_to_out, mi_stream stream) {
   if (!y || !w || !b || !out || rows < 0 || width < 1 || ldy < width || ldo < width) return MI_EINVAL;
@@ -1958,14 +2097,20 @@ static int launch_swa(const float* q, int64_t ldq, const void* kc, const void* v
     // prompt portions over a bf16 cache: the matrix-core form
     if (v16 && rows > n_seqs && D % 32 == 0 && Dv % 16 == 0 && D <= 256 && Dv <= 256 && ldv % 2 == 0) {
       const dim3 grid_m((((rows + 15) / 16) * H + 3) / 4);
-#define MI_SWA_MFMA(DKM, DVM, PAIR)                                                                                    \
-  hipLaunchKernelGGL((swa_attention_mfma_kernel<DKM, DVM, PAIR>), grid_m, dim3(256), 0, st, q, ldq, k, v, bt, cols, cu_q, \
-                     kv_lens, n_seqs, rows, H, G, D, Dv, block_size, window, scale, bias, ldv, gate, ldg, out, ldo)
+#define MI_SWA_MFMA(DKM, DVM, PAIR, KEEP)                                                                             \
+  hipLaunchKernelGGL((swa_attention_mfma_kernel<DKM, DVM, PAIR, KEEP>), grid_m, dim3(256), 0, st, q, ldq, k, v, bt, cols, \
+                     cu_q, kv_lens, n_seqs, rows, H, G, D, Dv, block_size, window, scale, bias, ldv, gate, ldg, out, ldo)
+#define MI_SWA_MFMA_KEEP(DKM, DVM, PAIR)                    \
+  do {                                                      \
+    if (bias.kept > 0) MI_SWA_MFMA(DKM, DVM, PAIR, true);   \
+    else MI_SWA_MFMA(DKM, DVM, PAIR, false);                \
+  } while (0)
       const bool small = D <= 128 && Dv <= 128, pair = Dv % 32 == 0;
-      if (small && pair) MI_SWA_MFMA(4, 8, true);
-      else if (small) MI_SWA_MFMA(4, 8, false);
-      else if (pair) MI_SWA_MFMA(8, 16, true);
-      else MI_SWA_MFMA(8, 16, false);
+      if (small && pair) MI_SWA_MFMA_KEEP(4, 8, true);
+      else if (small) MI_SWA_MFMA_KEEP(4, 8, false);
+      else if (pair) MI_SWA_MFMA_KEEP(8, 16, true);
+      else MI_SWA_MFMA_KEEP(8, 16, false);
+#undef MI_SWA_MFMA_KEEP
 #undef MI_SWA_MFMA
       return check_launch();
     }
@@ -1982,14 +2127,20 @@ static int launch_swa(const float* q, int64_t ldq, const void* kc, const void* v
         n_split *= 2;
       if (!ws) n_split = 1;
       const dim3 grid_h(rows, G, chunks * n_split);
-#define MI_HEADS_MFMA(DKM, DVM, PAIR)                                                                                  \
-  hipLaunchKernelGGL((paged_attention_heads_mfma_kernel<DKM, DVM, PAIR>), grid_h, dim3(256), 0, st, q, ldq, k, v, bt,   \
-                     cols, kv_lens, H, G, D, Dv, block_size, window, scale, bias, ldv, gate, ldg, out, ldo, n_split, ws)
+#define MI_HEADS_MFMA(DKM, DVM, PAIR, KEEP)                                                                           \
+  hipLaunchKernelGGL((paged_attention_heads_mfma_kernel<DKM, DVM, PAIR, KEEP>), grid_h, dim3(256), 0, st, q, ldq, k, v,  \
+                     bt, cols, kv_lens, H, G, D, Dv, block_size, window, scale, bias, ldv, gate, ldg, out, ldo, n_split, ws)
+#define MI_HEADS_MFMA_KEEP(DKM, DVM, PAIR)                    \
+  do {                                                        \
+    if (bias.kept > 0) MI_HEADS_MFMA(DKM, DVM, PAIR, true);   \
+    else MI_HEADS_MFMA(DKM, DVM, PAIR, false);                \
+  } while (0)
       const bool small = D <= 128 && Dv <= 128, pair = Dv % 32 == 0;
-      if (small && pair) MI_HEADS_MFMA(4, 8, true);
-      else if (small) MI_HEADS_MFMA(4, 8, false);
-      else if (pair) MI_HEADS_MFMA(8, 16, true);
-      else MI_HEADS_MFMA(8, 16, false);
+      if (small && pair) MI_HEADS_MFMA_KEEP(4, 8, true);
+      else if (small) MI_HEADS_MFMA_KEEP(4, 8, false);
+      else if (pair) MI_HEADS_MFMA_KEEP(8, 16, true);
+      else MI_HEADS_MFMA_KEEP(8, 16, false);
+#undef MI_HEADS_MFMA_KEEP
 #undef MI_HEADS_MFMA
       if (check_launch() != MI_OK) return MI_ELAUNCH;
       if (n_split == 1) return MI_OK;
@@ -2053,26 +2204,26 @@ extern "C" int mi_paged_attention_f32(const float* q, int64_t ldq, const void* k
                                       float* out, int64_t ldo, float* workspace, int64_t workspace_elems,
                                       mi_stream stream) {
   return mi_paged_attention_ext(q, ldq, k_cache, v_cache, ldv, cache_dtype, block_tables, table_cols, cu_q, kv_lens, n_seqs,
-                                rows, H, G, D, Dv, block_size, window, 0, scale, bias_kind, bias_p1, bias_p2, sink, 0.f, G,
+                                rows, H, G, D, Dv, block_size, window, 0, 0, scale, bias_kind, bias_p1, bias_p2, sink, 0.f, G,
                                 gate, ldg, out, ldo, workspace, workspace_elems, stream);
 }
 
 extern "C" int mi_paged_attention_ext(const float* q, int64_t ldq, const void* k_cache, const void* v_cache, int64_t ldv,
                                       int cache_dtype, const int32_t* block_tables, int table_cols, const int32_t* cu_q,
                                       const int32_t* kv_lens, int n_seqs, int rows, int H, int G, int D, int Dv,
-                                      int block_size, int window, int chunk, float scale, int bias_kind,
+                                      int block_size, int window, int chunk, int kept, float scale, int bias_kind,
                                       const float* bias_p1, const float* bias_p2, const float* sink, float softcap,
                                       int value_heads,
                                       const float* gate, int64_t ldg, float* out, int64_t ldo, float* workspace,
                                       int64_t workspace_elems, mi_stream stream) {
   if (!q || !k_cache || !v_cache || !block_tables || !cu_q || !kv_lens || !out || rows < 0 || n_seqs < 1) return MI_EINVAL;
   if (H < 1 || G < 1 || H % G || D < 1 || Dv < 1 || block_size < 1 || window < 1 || table_cols < 1 || ldv < Dv) return MI_EINVAL;
-  if (value_heads < 1 || G % value_heads || !(softcap >= 0.f) || chunk < 0) return MI_EINVAL;
+  if (value_heads < 1 || G % value_heads || !(softcap >= 0.f) || chunk < 0 || kept < 0) return MI_EINVAL;
   if (bias_kind != MI_BIAS_SLOPE && bias_kind != MI_BIAS_LOG && bias_kind != MI_BIAS_NONE) return MI_EINVAL;
   if (bias_kind == MI_BIAS_LOG && (!bias_p1 || !bias_p2)) return MI_EINVAL;
   if (Dv > 512 || D > 4096) return MI_EUNSUPPORTED;
   if (rows == 0) return MI_OK;
-  const AttnBias bias{bias_kind, bias_p1, bias_p2, sink, softcap, value_heads, chunk};
+  const AttnBias bias{bias_kind, bias_p1, bias_p2, sink, softcap, value_heads, chunk, kept};
   if (cache_dtype == MI_DTYPE_BF16)
     return launch_swa<uint16_t>(q, ldq, k_cache, v_cache, block_tables, table_cols, cu_q, kv_lens, n_seqs, rows, H, G, D,
                                 Dv, block_size, window, scale, bias, ldv, gate, ldg, out, ldo, workspace, workspace_elems,
@@ -2297,20 +2448,20 @@ extern "C" int mi_latent_prepare(const float* proj, int64_t ld, const float* q, 
   return check_launch();
 }
 
-extern "C" int mi_route_topk(const float* logits, int64_t ld, int n_tokens, int n_outputs, int top_k, int32_t* ids,
-                             float* weights, mi_stream stream) {
+extern "C" int mi_route_topk(const float* logits, int64_t ld, int n_tokens, int n_outputs, int top_k, float scale,
+                             int32_t* ids, float* weights, mi_stream stream) {
   if (!logits || !ids || !weights || n_tokens < 0 || ld < n_outputs) return MI_EINVAL;
   if (n_outputs < 1 || n_outputs > 512 || top_k < 1 || top_k > n_outputs) return MI_EUNSUPPORTED;
   if (n_tokens == 0) return MI_OK;
   hipLaunchKernelGGL(route_topk_kernel, dim3((n_tokens + 3) / 4), dim3(256), 0, S(stream), logits, ld, n_tokens, n_outputs,
-                     top_k, ids, weights);
+                     top_k, scale, ids, weights);
   return check_launch();
 }
 
 extern "C" int mi_moe_combine_shared(const float* y, const int32_t* ids, const float* weights, int n_tokens, int top_k,
                                      int width, const float* shared, int64_t ld_shared, const float* shared_gate,
                                      int64_t ld_gate, float* out, int64_t ldo, mi_stream stream) {
-  if (!y || !ids || !out || n_tokens < 0 || top_k < 1 || width < 1 || (shared && !shared_gate)) return MI_EINVAL;
+  if (!y || !ids || !out || n_tokens < 0 || top_k < 1 || width < 1) return MI_EINVAL;
   if (n_tokens == 0) return MI_OK;
   hipLaunchKernelGGL(moe_combine_shared_kernel, dim3(n_tokens), dim3(256), 0, S(stream), y, ids, weights, top_k, width,
                      shared, ld_shared, shared_gate, ld_gate, out, ldo);
@@ -2324,6 +2475,25 @@ extern "C" int mi_gated_norm_add_f32(float* res, int64_t ldr, const float* y, in
   if (rows == 0) return MI_OK;
   hipLaunchKernelGGL(gated_norm_add_f32_kernel, dim3(rows), dim3(256), 0, S(stream), res, ldr, y, ldy, gate_pre, ldg,
                      w_post, eps, w_next, out, ldo, width);
+  return check_launch();
+}
+
+extern "C" int mi_parts_norm_add_f32(float* res, int64_t ldr, const float* y, int parts, const float* weights,
+                                     const float* shared, int64_t ld_shared, const float* w_post, float eps,
+                                     const float* w_next, float* out, int64_t ldo, int rows, int width, mi_stream stream) {
+  if (!res || !y || !w_post || rows < 0 || width < 1 || parts < 1 || ldr < width || (shared && ld_shared < width) ||
+      (w_next && (!out || ldo < width)))
+    return MI_EINVAL;
+  if (rows == 0) return MI_OK;
+  const bool vec = width % 4 == 0 && ldr % 4 == 0 && aligned16(res) && aligned16(y) && aligned16(w_post) &&
+                   (!shared || (ld_shared % 4 == 0 && aligned16(shared))) &&
+                   (!w_next || (ldo % 4 == 0 && aligned16(out) && aligned16(w_next)));
+  if (vec)
+    hipLaunchKernelGGL(parts_norm_add_f32_kernel<4>, dim3(rows), dim3(256), 0, S(stream), res, ldr, y, parts, weights, shared,
+                       ld_shared, w_post, eps, w_next, out, ldo, width);
+  else
+    hipLaunchKernelGGL(parts_norm_add_f32_kernel<1>, dim3(rows), dim3(256), 0, S(stream), res, ldr, y, parts, weights, shared,
+                       ld_shared, w_post, eps, w_next, out, ldo, width);
   return check_launch();
 }
 
@@ -2380,13 +2550,14 @@ extern "C" int mi_linear_attention(const float* proj, int64_t ld, int q_off, int
 }
 
 extern "C" int mi_rotary_store(float* proj, int64_t ld, int q_off, int k_off, int v_off, int H, int G, int D, int Gv, int Dv,
-                               int rot_dims, int layout, const float* inv_freq, float amp, int unit_norm, float eps,
-                               float k_mult, const int32_t* cu_q, const int32_t* kv_lens, int n_seqs, void* k_cache,
+                               int rot_dims, int layout, const float* inv_freq, float amp, int unit_norm,
+                               const float* q_norm, const float* k_norm, float eps, float k_mult, const int32_t* cu_q, const int32_t* kv_lens, int n_seqs, void* k_cache,
                                void* v_cache, int cache_dtype, const int32_t* slots, int rows, int block_size,
                                mi_stream stream) {
   if (!proj || !cu_q || !kv_lens || rows < 0 || n_seqs < 1 || H < 0 || G < 0 || D < 1 || block_size < 1) return MI_EINVAL;
   if (rot_dims < 0 || rot_dims > D || rot_dims % 2 || (rot_dims && !inv_freq)) return MI_EINVAL;
   if (layout != MI_ROT_INTERLEAVED && layout != MI_ROT_HALVES) return MI_EINVAL;
+  if ((q_norm || k_norm) && !unit_norm) return MI_EINVAL;
   if ((k_cache || v_cache) && !slots) return MI_EINVAL;
   if (v_cache && (Gv < 1 || Dv < 1)) return MI_EINVAL;
   if (q_off + (int64_t)H * D > ld || k_off + (int64_t)G * D > ld || (v_cache && v_off + (int64_t)Gv * Dv > ld)) return MI_EINVAL;
@@ -2395,11 +2566,11 @@ extern "C" int mi_rotary_store(float* proj, int64_t ld, int q_off, int k_off, in
   if (rows == 0) return MI_OK;
   if (cache_dtype == MI_DTYPE_BF16)
     hipLaunchKernelGGL(rotary_store_kernel<uint16_t>, dim3(rows), dim3(256), lds, S(stream), proj, ld, q_off, k_off, v_off,
-                       H, G, D, Gv, Dv, rot_dims, layout, inv_freq, amp, unit_norm, eps, k_mult, cu_q, kv_lens, n_seqs,
+                       H, G, D, Gv, Dv, rot_dims, layout, inv_freq, amp, unit_norm, q_norm, k_norm, eps, k_mult, cu_q, kv_lens, n_seqs,
                        static_cast<uint16_t*>(k_cache), static_cast<uint16_t*>(v_cache), slots, block_size);
   else if (cache_dtype == MI_DTYPE_F32)
     hipLaunchKernelGGL(rotary_store_kernel<float>, dim3(rows), dim3(256), lds, S(stream), proj, ld, q_off, k_off, v_off, H,
-                       G, D, Gv, Dv, rot_dims, layout, inv_freq, amp, unit_norm, eps, k_mult, cu_q, kv_lens, n_seqs,
+                       G, D, Gv, Dv, rot_dims, layout, inv_freq, amp, unit_norm, q_norm, k_norm, eps, k_mult, cu_q, kv_lens, n_seqs,
                        static_cast<float*>(k_cache), static_cast<float*>(v_cache), slots, block_size);
   else
     return MI_EINVAL;

@@ -26,7 +26,7 @@ MI_OK = 0
 MI_EUNSUPPORTED = -2
 DTYPE_BF16, DTYPE_F32 = 0, 1
 ACT_NONE, ACT_SILU, ACT_GELU_TANH, ACT_GELU_ERF, ACT_SIGMOID, ACT_SOFTCAP, ACT_CLAMPED_GLU, ACT_TANH, \
-    ACT_DECAY = range(9)   # MI_ACT_*
+    ACT_DECAY, ACT_RELU2 = range(10)   # MI_ACT_*
 ROT_INTERLEAVED, ROT_HALVES = range(2)                                    # MI_ROT_*
 ROUTE_SOFTMAX, ROUTE_SIGMOID = range(2)                                   # MI_ROUTE_*
 ROUTE_GROUP_MAX, ROUTE_GROUP_TOP2 = range(2)                              # MI_ROUTE_GROUP_*
@@ -175,6 +175,7 @@ _SIGNATURES = {
     "mi_gemm_any_grouped": (c_int, [_p, c_int64, _p, _p, _p, c_int, _p, c_int, c_int, _p, c_int64, _p, c_int, c_int,
                                     c_int, _p]),
     "mi_embedding_f32": (c_int, [_p, _p, c_int, _p, c_int, c_int, c_int, c_float, _p]),
+    "mi_embedding_sinusoid_f32": (c_int, [_p, _p, c_int, _p, c_int, c_int, c_int, c_float, _p, _p, _p, c_int, _p]),
     "mi_layernorm_f32": (c_int, [_p, c_int64, _p, _p, _p, c_int64, c_int, c_int, c_float, c_int, _p]),
     "mi_swa_prepare": (c_int, [_p, c_int64, c_int, c_int, c_int, _p, _p, c_float, _p, c_int64, _p, _p, _p, c_int, _p,
                                c_int, c_int, c_int, c_int, c_int, c_int, _p]),
@@ -210,21 +211,22 @@ _SIGNATURES = {
                                  c_int, c_int, c_int, c_int, c_int, _p]),
     "mi_latent_prepare": (c_int, [_p, c_int64, _p, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _p, _p, c_float, _p,
                                   _p, c_int, _p, c_int, _p, _p, c_int64, c_int, _p]),
-    "mi_route_topk": (c_int, [_p, c_int64, c_int, c_int, c_int, _p, _p, _p]),
+    "mi_route_topk": (c_int, [_p, c_int64, c_int, c_int, c_int, c_float, _p, _p, _p]),
     "mi_moe_combine_shared": (c_int, [_p, _p, _p, c_int, c_int, c_int, _p, c_int64, _p, c_int64, _p, c_int64, _p]),
     "mi_gated_norm_add_f32": (c_int, [_p, c_int64, _p, c_int64, _p, c_int64, _p, c_float, _p, _p, c_int64, c_int, c_int, _p]),
+    "mi_parts_norm_add_f32": (c_int, [_p, c_int64, _p, c_int, _p, _p, c_int64, _p, c_float, _p, _p, c_int64, c_int, c_int, _p]),
     "mi_linear_attention_state_elems": (c_int64, [c_int, c_int, c_int]),
     "mi_linear_attention": (c_int, [_p, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _p, _p, _p, _p, c_int64,
                                     _p, c_int, _p, _p, _p, _p, c_int, c_int, c_int, c_int, c_int, c_float, _p, c_int64, _p]),
     "mi_paged_attention_ext": (c_int, [_p, c_int64, _p, _p, c_int64, c_int, _p, c_int, _p, _p, c_int, c_int, c_int, c_int,
-                                       c_int, c_int, c_int, c_int, c_int, c_float, c_int, _p, _p, _p, c_float, c_int, _p, c_int64,
+                                       c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, _p, _p, _p, c_float, c_int, _p, c_int64,
                                        _p, c_int64, _p, c_int64, _p]),
     "mi_add_vec_rmsnorm_f32": (c_int, [_p, c_int64, _p, c_int64, c_float, _p, _p, c_float, c_float, _p, c_int64, c_int, c_int,
                                        _p]),
     "mi_gemm_any_grouped_glu": (c_int, [_p, c_int64, _p, _p, _p, c_int, c_int, c_float, _p, _p, _p, c_int, c_int, _p, c_int64,
                                         _p, c_int, c_int, c_int, _p]),
     "mi_rotary_store": (c_int, [_p, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _p, c_float,
-                                c_int, c_float, c_float, _p, _p, c_int, _p, _p, c_int, _p, c_int, c_int, _p]),
+                                c_int, _p, _p, c_float, c_float, _p, _p, c_int, _p, _p, c_int, _p, c_int, c_int, _p]),
     "mi_head_mix": (c_int, [_p, c_int64, _p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, _p, c_int64, _p]),
     "mi_head_norm_gate": (c_int, [_p, c_int64, _p, c_int64, c_int, _p, c_int, c_float, c_int, c_int, c_int, c_float, _p]),
     "mi_gemm_any_segments": (c_int, [_p, c_int64, _p, c_int, _p, c_int, c_int, c_int, c_int, _p, c_int64, c_int, c_int, c_int,

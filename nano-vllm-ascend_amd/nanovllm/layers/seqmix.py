@@ -19,7 +19,7 @@ configuration:
                             query temperature, no rotation
   GatedDenseMLP             W_d (act(W_g h + b) * (W_u h + b)) + b
   SharedSparseMLP           top-k experts of the plain form W_d act(W_u h), softmax over the chosen logits, plus a shared
-                            expert behind a per-token sigmoid gate
+                            expert, behind a per-token sigmoid gate or as it is
   InputConvolution          what a sublayer reads is h + conv(h): a short causal depthwise convolution beside the identity,
                             its last taps - 1 inputs carried in the sequence's state slot
   GatedOutputNorm           a sublayer's output times sigmoid(W h + b) of the sublayer's input, RMS-normed, added to the
@@ -29,8 +29,8 @@ configuration:
   rotary_table              rotation frequencies of a head's channel pairs, optionally rescaled for long contexts (a ramp
                             between the fast pairs, kept, and the slow ones, divided by a factor; cos / sin amplified)
   RotaryWindowAttention     paged sliding-window attention over rotated (interleaved pairs) queries and keys, optionally
-                            behind short causal convolutions, with unit-normed heads, a sink logit per head, capped scores
-                            and mixing of the heads' softmax weights as options
+                            behind short causal convolutions, with normed heads, a sink, first tokens that stay visible,
+                            capped scores and mixing of the heads' softmax weights as options
   Retention                 linear attention over rotated (half-split pairs) queries and keys with a fixed decay per head,
                             per-head unit norm and a SiLU gate on the read-out
   SinkAttentionMixer        projections + RotaryWindowAttention + output projection
@@ -45,6 +45,11 @@ configuration:
   DifferentialAttention     two rotated softmax maps per head over the same values, a1 - lambda a2, unit-normed, with one
                             gate number per head; visibility within chunks of the sequence or causal
   GeneralDeltaMixer         generalised delta rule: channel-wise decay, removal along the unit key at a rate per channel
+  SinusoidEmbedding         scaled table rows plus sinusoids of the positions
+  OutputNorm                a sublayer's output, RMS-normed, added to the residual; the same launch sums an output that is
+                            still in parts (experts) and norms the stream for the next sublayer
+  PassInput                 what a pass over looped layers begins with: W [x | e] of the stream and the embedding output
+  DenseMLP                  W_d act(W_u h)
 
 Layers whose weights a model runs several times per step (a looped stack) keep one cache / state per pass ("lane"): their
 forward takes the lane's number.
@@ -214,7 +219,8 @@ class GroupedSparseMLP(nn.Module):
 # ---------------------------------------------------------------------------------------------------------------------
 # pre-norm families with a depth-mixed residual stream
 # ---------------------------------------------------------------------------------------------------------------------
-_ACTS = {"silu": _C.ACT_SILU, "gelu_tanh": _C.ACT_GELU_TANH, "gelu": _C.ACT_GELU_ERF, "sigmoid": _C.ACT_SIGMOID, None: _C.ACT_NONE}
+_ACTS = {"silu": _C.ACT_SILU, "gelu_tanh": _C.ACT_GELU_TANH, "gelu": _C.ACT_GELU_ERF, "sigmoid": _C.ACT_SIGMOID,
+         "relu2": _C.ACT_RELU2, None: _C.ACT_NONE}
 CAUSAL = 2 ** 31 - 1   # "window" of plain causal attention
 
 
@@ -375,32 +381,38 @@ class GatedDenseMLP(nn.Module):
 
 
 class SharedSparseMLP(nn.Module):
-    """Router logits in true 32-bit; the `top_k` largest, weights = softmax over them; experts W_d act(W_u h) without
-    biases; shared_ff > 0: a shared expert of the same form for every token, times sigmoid(w_sg . h) - that gate's row
-    rides behind the router's rows in one projection."""
+    """Router logits in true 32-bit; the `top_k` largest, weights = weight_scale * softmax over them; experts W_d act(W_u h)
+    without biases; shared_ff > 0: a shared expert of the same form for every token; shared_gate: times sigmoid(w_sg . h) -
+    that gate's row rides behind the router's rows in one projection."""
 
-    def __init__(self, width: int, ff: int, experts: int, top_k: int, shared_ff: int = 0, act: str = "gelu"):
+    def __init__(self, width: int, ff: int, experts: int, top_k: int, shared_ff: int = 0, act: str = "gelu",
+                 shared_gate: bool = True, weight_scale: float = 1.0):
         super().__init__()
         assert 1 <= top_k <= experts
-        self.E, self.top_k, self.act, self.shared = experts, top_k, _ACTS[act], shared_ff > 0
-        self.router = MergedRows(width, {"router": experts, "sg": 1} if self.shared else {"router": experts})
+        self.E, self.top_k, self.act, self.shared, self.weight_scale = experts, top_k, _ACTS[act], shared_ff > 0, weight_scale
+        self.gated = self.shared and shared_gate
+        self.router = MergedRows(width, {"router": experts, "sg": 1} if self.gated else {"router": experts})
         self.up, self.down = _matrix(experts, ff, width), _matrix(experts, width, ff)
         for p in (self.up, self.down):
             p.weight_loader = lambda param, tensor, expert: param.data[expert].copy_(tensor)
         if self.shared:
             self.shared_up, self.shared_down = _matrix(shared_ff, width), _matrix(width, shared_ff)
 
-    def forward(self, h: torch.Tensor) -> torch.Tensor:
+    def parts(self, h: torch.Tensor):
+        """-> (chosen experts' outputs [rows * top_k, width], their ids, their weights, shared expert's output | None, its
+        gate's pre-activation | None): the output before it is summed"""
         z = self.router(h, exact=True)
-        ids, wts = ops.route_topk(z, self.E, self.top_k)
+        ids, wts = ops.route_topk(z, self.E, self.top_k, self.weight_scale)
         offsets, pair_token, pair_index = ops.moe_sort(ids, self.E)
         P = ids.numel()
         a = ops.gemm_any_grouped_act(h, pair_token, self.up, None, self.act, offsets, P, None, P)
         y = ops.gemm_any_grouped_act(a, None, self.down, None, _C.ACT_NONE, offsets, P, pair_index, P)
-        if not self.shared:
-            return ops.moe_combine_shared(y, ids, wts, h.shape[1])
-        sh = ops.gemm_any(ops.gemm_any_act(h, self.shared_up, act=self.act), self.shared_down)
-        return ops.moe_combine_shared(y, ids, wts, h.shape[1], sh, z[:, self.E:])
+        sh = ops.gemm_any(ops.gemm_any_act(h, self.shared_up, act=self.act), self.shared_down) if self.shared else None
+        return y, ids, wts, sh, z[:, self.E:] if self.gated else None
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        y, ids, wts, shared, gate = self.parts(h)
+        return ops.moe_combine_shared(y, ids, wts, h.shape[1], shared, gate)
 
 
 # ---------------------------------------------------------------------------------------------------------------------
@@ -526,10 +538,12 @@ class RotaryWindowAttention(nn.Module):
     """The attention itself, on projections its owner made (`parts`: name -> rows of the q / k / v projections, to be laid
     out next to each other in this order).  conv_taps > 0: q, k and v first pass a causal convolution per channel (filters
     `conv.weight` [channels, taps], no activation), whose last taps - 1 inputs are the sequence's state.  Then q and k are
-    rotated (pairs 2i, 2i + 1 of the first rot_dims channels), unit_norm: each head divided by its root mean square;
-    s = scale q.k, softcap > 0: s <- softcap tanh(s / softcap); keys 0 <= i - j < window; softmax, sink: with
-    exp(sink_h) in the denominator; talk: the heads' weights are mixed, p'_h = sum_g talk[h, g] p_g, before head h applies
-    them to the values of its own key/value head.
+    rotated (pairs 2i, 2i + 1 of the first rot_dims channels), unit_norm: each head divided by its root mean square,
+    norm_weights: times a weight per channel, one for all query heads and one for all key heads;
+    s = scale q.k, softcap > 0: s <- softcap tanh(s / softcap); keys j <= i with i - j < window or j < keep_first (tokens
+    that stay visible); softmax, sink: with exp(sink_h) in the denominator - a parameter (True) or the same constant for
+    every head (a float); talk: the heads' weights are mixed, p'_h = sum_g talk[h, g] p_g, before head h applies them to the
+    values of its own key/value head.
 
     The mixing is linear in the weights, so it is done on read-outs: every query head's weights are applied to the values
     of ALL key/value heads (the value pages hold a token's heads side by side as ONE wide head, read in chunks of at most
@@ -537,16 +551,22 @@ class RotaryWindowAttention(nn.Module):
 
     def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, window: int, scale: float, eps: float,
                  rot_dims: int, rot_base: float, rot_scaling: dict | None = None, unit_norm: bool = False,
-                 sink: bool = False, softcap: float = 0.0, conv_taps: int = 0, talk: bool = False):
+                 sink: bool | float = False, softcap: float = 0.0, conv_taps: int = 0, talk: bool = False,
+                 norm_weights: bool = False, keep_first: int = 0):
         super().__init__()
         assert heads % kv_heads == 0 and 0 <= rot_dims <= dim and rot_dims % 2 == 0
+        assert window >= 1 and keep_first >= 0 and (unit_norm or not norm_weights)
         self.H, self.G, self.D, self.Dv = heads, kv_heads, dim, vdim
         self.window, self.scale, self.eps, self.unit_norm, self.softcap = window, scale, eps, unit_norm, softcap
-        self.rot_dims = rot_dims
+        self.rot_dims, self.keep_first = rot_dims, keep_first
         freq, self.rot_amp = rotary_table(rot_dims, rot_base, rot_scaling) if rot_dims else (torch.zeros(1, dtype=torch.float32), 1.0)
         self.register_buffer("inv_freq", freq, persistent=False)
         self.parts = {"q": heads * dim, "k": kv_heads * dim, "v": kv_heads * vdim}
-        self.sink = _vector(heads) if sink else None
+        self.q_norm, self.k_norm = (_vector(dim, 1.0), _vector(dim, 1.0)) if norm_weights else (None, None)
+        if isinstance(sink, bool):
+            self.sink = _vector(heads) if sink else None
+        else:   # (a buffer, not a checkpoint tensor)
+            self.register_buffer("sink", torch.full((heads,), float(sink), dtype=torch.float32), persistent=False)
         self.talk = nn.Parameter(torch.eye(heads, dtype=torch.float32), requires_grad=False) if talk else None
         self.conv = MergedRows(conv_taps, self.parts, dtype=torch.float32) if conv_taps else None
         self.k_cache, self.v_cache, self.conv_state = [], [], []   # one per lane
@@ -576,12 +596,13 @@ class RotaryWindowAttention(nn.Module):
         k_off, v_off = q_off + H * D, q_off + H * D + G * D
         kc, vc = self.k_cache[lane], self.v_cache[lane]
         ops.rotary_store(y, q_off, k_off, v_off, H, G, D, self.rot_dims, _C.ROT_INTERLEAVED, self.inv_freq, self.rot_amp,
-                         self.unit_norm, self.eps, 1.0, ctx.cu_seqlens_q, ctx.kv_lens, kc, vc, ctx.slot_mapping, ctx.block_size)
+                         self.unit_norm, self.eps, 1.0, ctx.cu_seqlens_q, ctx.kv_lens, kc, vc, ctx.slot_mapping, ctx.block_size,
+                         q_norm=self.q_norm, k_norm=self.k_norm)
         q = y[:, q_off:q_off + H * D]
         if self.talk is None:
             ops.paged_attention_f32(q, kc, vc, Dv, ctx.block_tables, ctx.cu_seqlens_q, ctx.kv_lens, H, G, D, Dv,
                                     ctx.block_size, self.window, self.scale, _C.BIAS_NONE, sink=self.sink,
-                                    softcap=self.softcap, out=out)
+                                    softcap=self.softcap, kept=self.keep_first, out=out)
             if out_scale != 1.0:
                 out.mul_(out_scale)
             return
@@ -589,7 +610,7 @@ class RotaryWindowAttention(nn.Module):
             nc = min(self.chunk, G - c0)
             o = ops.paged_attention_f32(q, kc, vc, G * Dv, ctx.block_tables, ctx.cu_seqlens_q, ctx.kv_lens, H, G, D, nc * Dv,
                                         ctx.block_size, self.window, self.scale, _C.BIAS_NONE, sink=self.sink,
-                                        softcap=self.softcap, value_heads=1, v_offset=c0 * Dv)
+                                        softcap=self.softcap, value_heads=1, v_offset=c0 * Dv, kept=self.keep_first)
             ops.head_mix(o, self.talk, H, G, Dv, c0, nc, out, out_scale)
 
 
@@ -846,3 +867,71 @@ class GeneralDeltaMixer(nn.Module):
                               ctx.state_slots, self.H, self.D, self.D)
         ops.head_norm_gate(o, m.cols(y, "g"), _C.ACT_SIGMOID, self.norm, self.H, self.D, self.eps)
         return ops.gemm_any(o, self.o)
+
+
+# ---------------------------------------------------------------------------------------------------------------------
+# sandwich-normed looped families: positions in the embedding, ungated output norms, a projection at every pass's beginning
+# ---------------------------------------------------------------------------------------------------------------------
+class SinusoidEmbedding(nn.Module):
+    """scale * E[token] + s, s[2i] = sin(t f_i), s[2i + 1] = cos(t f_i), f_i = base^(-2 i / width) (fp32 rows)."""
+
+    def __init__(self, vocab: int, width: int, scale: float, base: float = 10000.0):
+        super().__init__()
+        self.scale = scale
+        self.weight = _matrix(vocab, width)
+        f = [float(base) ** (-2.0 * i / width) for i in range((width + 1) // 2)]   # (double, rounded once)
+        self.register_buffer("inv_freq", torch.tensor(f, dtype=torch.float64).to(torch.float32), persistent=False)
+
+    def forward(self, ids: torch.Tensor) -> torch.Tensor:
+        ctx = get_context()
+        return ops.embedding_sinusoid_f32(ids, self.weight, self.scale, self.inv_freq, ctx.cu_seqlens_q, ctx.kv_lens)
+
+
+class OutputNorm(nn.Module):
+    """x <- x + rms(y) * w for a sublayer's output y."""
+
+    def __init__(self, width: int, eps: float):
+        super().__init__()
+        self.eps, self.weight = eps, _vector(width, 1.0)
+
+    def add_to(self, residual: torch.Tensor, y: torch.Tensor, next_norm: torch.Tensor | None):
+        """residual += rms(y) * w in place; -> rms(residual) * next_norm (None without one)"""
+        return ops.parts_norm_add_f32(residual, y, self.weight, self.eps, w_next=next_norm)
+
+    def add_experts_to(self, residual: torch.Tensor, mlp: SharedSparseMLP, h: torch.Tensor, next_norm: torch.Tensor | None):
+        """the same for y = mlp(h), whose parts are summed in the same launch (an ungated shared expert)"""
+        assert not mlp.gated
+        y, _, wts, shared, _ = mlp.parts(h)
+        return ops.parts_norm_add_f32(residual, y, self.weight, self.eps, wts=wts, shared=shared, w_next=next_norm)
+
+
+class PassInput(nn.Module):
+    """x <- W [x | e] = W_x x + W_e e.  W_e e is the same in every pass of a step: `fixed_part` once, `begin` per pass."""
+
+    def __init__(self, width: int):
+        super().__init__()
+        self.weight = _matrix(2, width, width)   # W_x, W_e: the column halves of the checkpoint's [width, 2 width]
+
+        def load(param, tensor):
+            assert tensor.shape == (width, 2 * width), tuple(tensor.shape)
+            param.data[0].copy_(tensor[:, :width])
+            param.data[1].copy_(tensor[:, width:])
+        self.weight.weight_loader = load
+
+    def fixed_part(self, e: torch.Tensor) -> torch.Tensor:
+        return ops.gemm_any(e, self.weight[1])
+
+    def begin(self, x: torch.Tensor, fixed: torch.Tensor, norm_w: torch.Tensor, eps: float):
+        """-> (the new stream, its norm with norm_w)"""
+        x = ops.gemm_any(x, self.weight[0])
+        return x, ops.add_rmsnorm_f32(x, fixed, 1.0, norm_w, eps)
+
+
+class DenseMLP(nn.Module):
+    def __init__(self, width: int, ff: int, act: str = "gelu_tanh"):
+        super().__init__()
+        self.act = _ACTS[act]
+        self.up, self.down = _matrix(ff, width), _matrix(width, ff)
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        return ops.gemm_any(ops.gemm_any_act(h, self.up, act=self.act), self.down)

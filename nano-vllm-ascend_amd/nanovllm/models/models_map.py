@@ -9,6 +9,7 @@ from nanovllm.models.munizen import MunizenConfig, MunizenForCausalLM
 from nanovllm.models.qwen3 import Qwen3ForCausalLM
 from nanovllm.models.qwen3_moe import Qwen3MoeForCausalLM
 from nanovllm.models.sanevik import SanevikConfig, SanevikForCausalLM
+from nanovllm.models.sikevik import SikevikConfig, SikevikForCausalLM
 from nanovllm.models.zedirax import ZediraxConfig, ZediraxForCausalLM
 
 model_dict = {
@@ -21,6 +22,7 @@ model_dict = {
     "Felolorn": FelolornForCausalLM,
     "Sanevik": SanevikForCausalLM,
     "Munizen": MunizenForCausalLM,
+    "Sikevik": SikevikForCausalLM,
 }
 
 # designs whose config.json is not a transformers configuration: {"architecture": <name>, ...} -> the reader of it
@@ -30,6 +32,7 @@ native_configs = {
     "Felolorn": FelolornConfig,
     "Sanevik": SanevikConfig,
     "Munizen": MunizenConfig,
+    "Sikevik": SikevikConfig,
 }
 
 

@@ -996,6 +996,21 @@ def embedding_f32(ids, table, out=None, scale: float = 1.0) -> torch.Tensor:
     return out
 
 
+def embedding_sinusoid_f32(ids, table, scale: float, inv_freq, cu_q, kv_lens) -> torch.Tensor:
+    """table[ids] * scale + sinusoids of the rows' positions: sin(pos * inv_freq[i]) on channel 2i, cos on channel 2i + 1."""
+    require_gpu(ids, table, inv_freq, cu_q, kv_lens)
+    _f32(inv_freq)
+    _i32(cu_q, kv_lens)
+    V, W = table.shape
+    assert ids.dtype == torch.int64 and ids.is_contiguous() and table.is_contiguous()
+    assert inv_freq.is_contiguous() and inv_freq.numel() >= (W + 1) // 2 and cu_q.numel() == kv_lens.numel() + 1
+    out = torch.empty((ids.numel(), W), dtype=_F32, device=table.device)
+    check(lib.mi_embedding_sinusoid_f32(ptr(ids), ptr(table), _dt(table), ptr(out), ids.numel(), W, V, float(scale),
+                                        ptr(inv_freq), ptr(cu_q), ptr(kv_lens), kv_lens.numel(), stream()),
+          "mi_embedding_sinusoid_f32")
+    return out
+
+
 def layernorm_f32(y, w, b, eps: float, add_to=None) -> torch.Tensor:
     """LN(y) * w + b per row; add_to: the residual it is added to IN PLACE (returned)."""
     require_gpu(y, w, b)
@@ -1204,10 +1219,11 @@ def gemm_any_batched(x, x_batch: int, w, out, out_batch: int, gate=None, gate_ba
 def paged_attention_f32(q, k_cache, v_cache, ldv: int, block_tables, cu_q, kv_lens, H: int, G: int, D: int, Dv: int,
                         block_size: int, window: int, scale: float, bias_kind: int = _C.BIAS_NONE, bias_p1=None, bias_p2=None,
                         gate=None, sink=None, softcap: float = 0.0, value_heads: int | None = None,
-                        v_offset: int = 0, chunk: int = 0, out=None) -> torch.Tensor:
+                        v_offset: int = 0, chunk: int = 0, kept: int = 0, out=None) -> torch.Tensor:
     """Paged causal attention over fp32 queries; see mi_paged_attention_ext (bias kinds, values inside the key rows, a
     sink logit per head in the softmax's denominator, capped scores, fewer and wider value heads than key heads with the
-    value rows read from column v_offset on, visibility within chunks of `chunk` positions)."""
+    value rows read from column v_offset on, visibility within chunks of `chunk` positions, the first `kept` keys of a
+    sequence visible whatever window and chunk say)."""
     require_gpu(q, k_cache, v_cache, block_tables, cu_q, kv_lens)
     _f32(q, gate, bias_p1, bias_p2, sink)
     assert sink is None or (sink.numel() == H and sink.is_contiguous())
@@ -1226,7 +1242,7 @@ def paged_attention_f32(q, k_cache, v_cache, ldv: int, block_tables, cu_q, kv_le
     check(lib.mi_paged_attention_ext(ptr(q), q.stride(0), ptr(k_cache), ptr(v_cache) + v_offset * v_cache.element_size(),
                                      int(ldv), _dt(k_cache),
                                      ptr(block_tables), block_tables.shape[1], ptr(cu_q), ptr(kv_lens), n_seqs, rows, H, G,
-                                     D, Dv, block_size, int(min(window, 2 ** 31 - 1)), int(chunk), float(scale), int(bias_kind),
+                                     D, Dv, block_size, int(min(window, 2 ** 31 - 1)), int(chunk), int(kept), float(scale), int(bias_kind),
                                      ptr(bias_p1), ptr(bias_p2), ptr(sink), float(softcap),
                                      int(G if value_heads is None else value_heads), ptr(gate),
                                      gate.stride(0) if gate is not None else 0,
@@ -1315,26 +1331,27 @@ def latent_prepare(proj, q, q_off: int, c_off: int, H: int, D: int, R: int, C: i
                                 ptr(slots), ptr(qx), qx.stride(0), rows, stream()), "mi_latent_prepare")
 
 
-def route_topk(logits, n_outputs: int, top_k: int):
-    """The top_k largest of the first n_outputs columns; weights = softmax over the chosen logits."""
+def route_topk(logits, n_outputs: int, top_k: int, scale: float = 1.0):
+    """The top_k largest of the first n_outputs columns; weights = scale * softmax over the chosen logits."""
     require_gpu(logits)
     _f32(logits)
     T = logits.shape[0]
     assert n_outputs <= logits.shape[1]
     ids = torch.empty((T, top_k), dtype=torch.int32, device=logits.device)
     wts = torch.empty((T, top_k), dtype=_F32, device=logits.device)
-    check(lib.mi_route_topk(ptr(logits), logits.stride(0), T, n_outputs, top_k, ptr(ids), ptr(wts), stream()),
-          "mi_route_topk")
+    check(lib.mi_route_topk(ptr(logits), logits.stride(0), T, n_outputs, top_k, float(scale), ptr(ids), ptr(wts),
+                            stream()), "mi_route_topk")
     return ids, wts
 
 
 def moe_combine_shared(y, ids, wts, width: int, shared=None, shared_gate=None) -> torch.Tensor:
-    """sum_k wts[t][k] * y[t * top_k + k] (+ sigmoid(shared_gate[t]) * shared[t]); wts None: every weight 1."""
+    """sum_k wts[t][k] * y[t * top_k + k] (+ sigmoid(shared_gate[t]) * shared[t], without a gate shared[t] itself); wts
+    None: every weight 1."""
     require_gpu(y, ids)
     _f32(y, wts, shared)
     T, top_k = ids.shape
     assert y.shape == (T * top_k, width) and y.is_contiguous()
-    assert shared is None or (shared.shape == (T, width) and shared_gate is not None and shared_gate.dtype == _F32)
+    assert shared is None or (shared.shape == (T, width) and (shared_gate is None or shared_gate.dtype == _F32))
     out = torch.empty((T, width), dtype=_F32, device=y.device)
     check(lib.mi_moe_combine_shared(ptr(y), ptr(ids), ptr(wts), T, top_k, width, ptr(shared),
                                     shared.stride(0) if shared is not None else 0, ptr(shared_gate),
@@ -1359,6 +1376,26 @@ def gated_norm_add_f32(res, y, gate_pre, w_post, eps: float, w_next=None):
     check(lib.mi_gated_norm_add_f32(ptr(res), res.stride(0), ptr(y), y.stride(0), ptr(gate_pre),
                                     gate_pre.stride(0) if gate_pre is not None else 0, ptr(w_post), float(eps), ptr(w_next),
                                     ptr(out), width, rows, width, stream()), "mi_gated_norm_add_f32")
+    return out
+
+
+def parts_norm_add_f32(res, y, w_post, eps: float, wts=None, shared=None, w_next=None):
+    """v = sum_k wts[t][k] * y[t * parts + k] + shared[t] (wts None: ones, shared None: nothing; y [rows * parts, width]);
+    res += rms(v) * w_post in place; w_next given: returns rms(res) * w_next, else None."""
+    require_gpu(res, y, w_post)
+    _f32(res, y, wts, shared, w_post, w_next)
+    rows, width = res.shape
+    parts = y.shape[0] // max(rows, 1)
+    assert y.is_contiguous() and y.shape == (rows * parts, width) and w_post.numel() == width
+    assert wts is None or (wts.is_contiguous() and wts.numel() == rows * parts)
+    assert shared is None or shared.shape == res.shape
+    out = None
+    if w_next is not None:
+        assert w_next.numel() == width
+        out = torch.empty((rows, width), dtype=_F32, device=res.device)
+    check(lib.mi_parts_norm_add_f32(ptr(res), res.stride(0), ptr(y), parts, ptr(wts), ptr(shared),
+                                    shared.stride(0) if shared is not None else 0, ptr(w_post), float(eps), ptr(w_next),
+                                    ptr(out), width, rows, width, stream()), "mi_parts_norm_add_f32")
     return out
 
 
@@ -1421,12 +1458,14 @@ def gemm_any_grouped_glu(x, x_rows, w, w2, act: int, limit: float, row_scale, ro
 
 def rotary_store(proj, q_off: int, k_off: int, v_off: int, H: int, G: int, D: int, rot_dims: int, layout: int, inv_freq,
                  amp: float, unit_norm: bool, eps: float, k_mult: float, cu_q, kv_lens, k_cache=None, v_cache=None, slots=None,
-                 block_size: int = 1) -> None:
+                 block_size: int = 1, q_norm=None, k_norm=None) -> None:
     """Rotates the H query and G key heads of every row of proj in place (see mi_rotary_store); with caches the key heads
-    go to k_cache [blocks, G, block_size, D] and the row's values at v_off to v_cache [blocks, Gv, block_size, Dv]."""
+    go to k_cache [blocks, G, block_size, D] and the row's values at v_off to v_cache [blocks, Gv, block_size, Dv]; q_norm /
+    k_norm [D]: weights of the heads' norm (with unit_norm)."""
     require_gpu(proj, k_cache, v_cache, slots)
-    _f32(proj, inv_freq)
+    _f32(proj, inv_freq, q_norm, k_norm)
     _i32(cu_q, kv_lens, slots)
+    assert (q_norm is None or q_norm.numel() == D) and (k_norm is None or k_norm.numel() == D)
     rows = proj.shape[0]
     Gv = Dv = 0
     dt = _C.DTYPE_F32
@@ -1440,7 +1479,8 @@ def rotary_store(proj, q_off: int, k_off: int, v_off: int, H: int, G: int, D: in
     assert slots is None or slots.numel() == rows
     assert rot_dims == 0 or (inv_freq.is_cuda and inv_freq.numel() >= rot_dims // 2)
     check(lib.mi_rotary_store(ptr(proj), proj.stride(0), q_off, k_off, v_off, H, G, D, Gv, Dv, int(rot_dims), int(layout),
-                              ptr(inv_freq), float(amp), int(unit_norm), float(eps), float(k_mult), ptr(cu_q), ptr(kv_lens),
+                              ptr(inv_freq), float(amp), int(unit_norm), ptr(q_norm), ptr(k_norm), float(eps), float(k_mult), ptr(cu_q),
+                              ptr(kv_lens),
                               kv_lens.numel(), ptr(k_cache), ptr(v_cache), dt, ptr(slots), rows, block_size, stream()),
           "mi_rotary_store")
 
