@@ -1,5 +1,5 @@
 """Prefill and decode throughput of a model design beside the framework's closest existing model at equal size
-(`python bench.py --design gazutar | zedirax | felolorn | sanevik | munizen`): random weights, layer sizes that resemble a real model's, both models through the same
+(`python bench.py --design gazutar | zedirax | felolorn | sanevik | munizen | sikevik`): random weights, layer sizes that resemble a real model's, both models through the same
 engine entry points (add_request / step), each served the way the framework serves it (Qwen3-MoE: captured prefill and
 decode steps; Gazutar: what ModelRunner reports in `served_as`).
 
@@ -183,6 +183,38 @@ def munizen_decode_weight_bytes(cfg: dict) -> float:
     return 2.0 * (n + cfg["vocab"] * W)
 
 
+def sikevik_config(s: dict) -> dict:
+    """Four window attentions whose first 16 tokens stay visible, the first with a dense feed-forward as wide as the experts a
+    token visits, the others with sparse ones and a shared expert of one expert's size; the last two layers run twice (six
+    layer runs per step, each with pages of its own)."""
+    W, D = s["width"], s["dim"]
+    att = {"type": "attention", "mixer": {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": D, "vdim": D, "scale": D ** -0.5,
+                                          "mask": {"size": s["window"], "keep_first": 16}}}
+    dense = {"kind": "dense", "ff": s["top"] * s["ff"]}
+    moe = {"kind": "moe", "expert": {"ff": s["ff"]}, "router": {"experts": s["experts"], "top": s["top"], "scale": 2.0},
+           "shared": {"ff": s["ff"]}}
+    n = s["layers"]
+    return {"architecture": "Sikevik", "vocab": s["vocab"], "width": W, "norm": {"eps": 1e-6}, "embedding": {"scale": W ** 0.5},
+            "loop": {"start": n - 2, "stop": n, "times": 2}, "layers": [dict(att, mlp=moe if i else dense) for i in range(n)]}
+
+
+def sikevik_decode_weight_bytes(cfg: dict, batch: int) -> float:
+    """bf16 weight bytes a decode step streams: every projection and the experts the rows can reach, once per RUN of a layer,
+    the projection at a pass's beginning (its embedding half once), the tied table as the head."""
+    W, loop = cfg["width"], cfg["loop"]
+    n = W * W * (loop["times"] + 1)
+    for i, l in enumerate(cfg["layers"]):
+        m, ml = l["mixer"], l["mlp"]
+        mix = W * (m["heads"] * m["dim"] + m["kv_heads"] * (m["dim"] + m["vdim"])) + m["heads"] * m["vdim"] * W
+        if ml["kind"] == "dense":
+            mix += 2 * W * ml["ff"]
+        else:
+            hit = min(ml["router"]["experts"], batch * ml["router"]["top"])
+            mix += hit * 2 * W * ml["expert"]["ff"] + ml["router"]["experts"] * W + 2 * W * ml["shared"]["ff"]
+        n += mix * (loop["times"] if loop["start"] <= i < loop["stop"] else 1)
+    return 2.0 * (n + cfg["vocab"] * W)
+
+
 def qwen3_moe_config(s: dict) -> dict:
     return dict(architectures=["Qwen3MoeForCausalLM"], model_type="qwen3_moe", hidden_size=s["width"],
                 num_hidden_layers=s["layers"], num_attention_heads=s["heads"], num_key_value_heads=s["kv_heads"],
@@ -264,6 +296,8 @@ def main(args) -> dict:
         return main_sanevik(args, batch, prompt_len)
     if design == "munizen":
         return main_munizen(args, batch, prompt_len)
+    if design == "sikevik":
+        return main_sikevik(args, batch, prompt_len)
     out = {"metric": "design_throughput", "design": "gazutar", "closest_model": "Qwen3MoeForCausalLM", "unit": "tokens/s",
            "dtype": "bf16", "data": "synthetic (random weights, random prompts)", "n_gpus": 1, "steps": args.steps,
            "warmup": args.warmup, "batch": batch, "prompt_len": prompt_len, "sizes": {}}
@@ -351,72 +385,78 @@ def main_felolorn(args, batch: int, prompt_len: int) -> dict:
     return out
 
 
+def _beside(args, batch: int, prompt_len: int, design: str, closest: str, models, others, default) -> dict:
+    """The record of a looped design beside other models: models(size) -> [(label, config, weight bytes of a decode step, layer
+    runs)]; rates relative to each of `others`, per step and per layer run (a looped layer counts once per pass)."""
+    out = {"metric": "design_throughput", "design": design, "closest_model": closest, "unit": "tokens/s",
+           "dtype": "bf16", "data": "synthetic (random weights, random prompts)", "n_gpus": 1, "steps": args.steps,
+           "warmup": args.warmup, "batch": batch, "prompt_len": prompt_len, "sizes": {}}
+    only_sizes = [x for x in getattr(args, "design_sizes", "").split(",") if x]
+    only_models = [x for x in getattr(args, "design_models", "").split(",") if x] or default
+    for name, s in SIZES.items():
+        if only_sizes and name not in only_sizes:
+            continue
+        entry = {"shape": s}
+        for label, cfg, wb, runs in models(s):
+            if label not in only_models:
+                continue
+            r = run_model(cfg, batch, prompt_len, args.steps, args.warmup)
+            r["layer_runs"] = runs
+            r["decode_weight_bytes"] = wb
+            r["decode_weight_roofline_frac"] = wb / (r["ms_per_decode_step"] * 1e-3) / HBM_BYTES_PER_S
+            entry[label] = r
+        for other in others:
+            if design in entry and other in entry:
+                key = f"{design}_vs_{other}"
+                entry[key] = {k: entry[design][k] / entry[other][k] for k in ("prefill_tok_s", "decode_tok_s")}
+                entry[key + "_per_layer_run"] = {
+                    k: v * entry[design]["layer_runs"] / entry[other]["layer_runs"] for k, v in entry[key].items()}
+        out["sizes"][name] = entry
+    print(json.dumps(out), flush=True)
+    return out
+
+
 def main_sanevik(args, batch: int, prompt_len: int) -> dict:
     """Sanevik beside Gazutar - the closest existing model: the same row-step engine path, fp32 residual, sliding-window
     attention over paged K / V rows alternating with a matrix-state recurrence behind short convolutions, sparse
     feed-forwards - at equal width, depth, heads, experts and vocabulary; Felolorn (sink softmax, head-decay linear
     attention) and Qwen3-MoE at that size ride along (`--design-models` picks).  Sanevik runs its last two layers twice:
     six layer runs per step against the others' four (`layer_runs` in the record)."""
-    out = {"metric": "design_throughput", "design": "sanevik", "closest_model": "Gazutar", "unit": "tokens/s",
-           "dtype": "bf16", "data": "synthetic (random weights, random prompts)", "n_gpus": 1, "steps": args.steps,
-           "warmup": args.warmup, "batch": batch, "prompt_len": prompt_len, "sizes": {}}
-    only_sizes = [x for x in getattr(args, "design_sizes", "").split(",") if x]
-    only_models = [x for x in getattr(args, "design_models", "").split(",") if x] or ["sanevik", "gazutar", "felolorn"]
-    for name, s in SIZES.items():
-        if only_sizes and name not in only_sizes:
-            continue
-        entry = {"shape": s}
+    def models(s):
         sc, fc = sanevik_config(s), felolorn_config(s)
-        for label, cfg, wb, runs in (("sanevik", sc, sanevik_decode_weight_bytes(sc, batch), s["layers"] + 2),
-                                     ("gazutar", gazutar_config(s), decode_weight_bytes(s, batch, True), s["layers"]),
-                                     ("felolorn", fc, felolorn_decode_weight_bytes(fc, batch), s["layers"]),
-                                     ("qwen3_moe", qwen3_moe_config(s), decode_weight_bytes(s, batch, False), s["layers"])):
-            if label not in only_models:
-                continue
-            r = run_model(cfg, batch, prompt_len, args.steps, args.warmup)
-            r["layer_runs"] = runs
-            r["decode_weight_bytes"] = wb
-            r["decode_weight_roofline_frac"] = wb / (r["ms_per_decode_step"] * 1e-3) / HBM_BYTES_PER_S
-            entry[label] = r
-        for other in ("gazutar", "felolorn"):
-            if "sanevik" in entry and other in entry:
-                entry["sanevik_vs_" + other] = {k: entry["sanevik"][k] / entry[other][k] for k in ("prefill_tok_s", "decode_tok_s")}
-                entry["sanevik_vs_" + other + "_per_layer_run"] = {
-                    k: v * entry["sanevik"]["layer_runs"] / entry[other]["layer_runs"] for k, v in entry["sanevik_vs_" + other].items()}
-        out["sizes"][name] = entry
-    print(json.dumps(out), flush=True)
-    return out
+        return [("sanevik", sc, sanevik_decode_weight_bytes(sc, batch), s["layers"] + 2),
+                ("gazutar", gazutar_config(s), decode_weight_bytes(s, batch, True), s["layers"]),
+                ("felolorn", fc, felolorn_decode_weight_bytes(fc, batch), s["layers"]),
+                ("qwen3_moe", qwen3_moe_config(s), decode_weight_bytes(s, batch, False), s["layers"])]
+
+    return _beside(args, batch, prompt_len, "sanevik", "Gazutar", models, ("gazutar", "felolorn"),
+                   ["sanevik", "gazutar", "felolorn"])
 
 
 def main_munizen(args, batch: int, prompt_len: int) -> dict:
     """Munizen beside Gazutar - the closest existing model: the same row-step engine path, fp32 residual, a delta rule with a
     decay per key channel alternating with windowed attention - at equal width, depth, heads and vocabulary; Sanevik (looped,
     rotated heads) rides along (`--design-models` picks).  `layer_runs` counts a looped layer once per pass."""
-    out = {"metric": "design_throughput", "design": "munizen", "closest_model": "Gazutar", "unit": "tokens/s",
-           "dtype": "bf16", "data": "synthetic (random weights, random prompts)", "n_gpus": 1, "steps": args.steps,
-           "warmup": args.warmup, "batch": batch, "prompt_len": prompt_len, "sizes": {}}
-    only_sizes = [x for x in getattr(args, "design_sizes", "").split(",") if x]
-    only_models = [x for x in getattr(args, "design_models", "").split(",") if x] or ["munizen", "gazutar", "sanevik"]
-    for name, s in SIZES.items():
-        if only_sizes and name not in only_sizes:
-            continue
-        entry = {"shape": s}
+    def models(s):
         mc, sc = munizen_config(s), sanevik_config(s)
-        for label, cfg, wb, runs in (("munizen", mc, munizen_decode_weight_bytes(mc), s["layers"] + 2),
-                                     ("gazutar", gazutar_config(s), decode_weight_bytes(s, batch, True), s["layers"]),
-                                     ("sanevik", sc, sanevik_decode_weight_bytes(sc, batch), s["layers"] + 2)):
-            if label not in only_models:
-                continue
-            r = run_model(cfg, batch, prompt_len, args.steps, args.warmup)
-            r["layer_runs"] = runs
-            r["decode_weight_bytes"] = wb
-            r["decode_weight_roofline_frac"] = wb / (r["ms_per_decode_step"] * 1e-3) / HBM_BYTES_PER_S
-            entry[label] = r
-        for other in ("gazutar", "sanevik"):
-            if "munizen" in entry and other in entry:
-                entry["munizen_vs_" + other] = {k: entry["munizen"][k] / entry[other][k] for k in ("prefill_tok_s", "decode_tok_s")}
-                entry["munizen_vs_" + other + "_per_layer_run"] = {
-                    k: v * entry["munizen"]["layer_runs"] / entry[other]["layer_runs"] for k, v in entry["munizen_vs_" + other].items()}
-        out["sizes"][name] = entry
-    print(json.dumps(out), flush=True)
-    return out
+        return [("munizen", mc, munizen_decode_weight_bytes(mc), s["layers"] + 2),
+                ("gazutar", gazutar_config(s), decode_weight_bytes(s, batch, True), s["layers"]),
+                ("sanevik", sc, sanevik_decode_weight_bytes(sc, batch), s["layers"] + 2)]
+
+    return _beside(args, batch, prompt_len, "munizen", "Gazutar", models, ("gazutar", "sanevik"), ["munizen", "gazutar", "sanevik"])
+
+
+def main_sikevik(args, batch: int, prompt_len: int) -> dict:
+    """Sikevik beside Sanevik - the closest existing model: the same row-step engine path, fp32 residual, a looped stack with
+    pages per pass, window attention with a sink over normed heads, sparse feed-forwards - at equal width, depth, heads,
+    experts, vocabulary and layer runs; Zedirax (plain experts beside a shared one) and Gazutar (window attention) ride along
+    (`--design-models` picks)."""
+    def models(s):
+        kc, sc, zc = sikevik_config(s), sanevik_config(s), zedirax_config(s)
+        return [("sikevik", kc, sikevik_decode_weight_bytes(kc, batch), s["layers"] + 2),
+                ("sanevik", sc, sanevik_decode_weight_bytes(sc, batch), s["layers"] + 2),
+                ("zedirax", zc, zedirax_decode_weight_bytes(zc, batch), s["layers"]),
+                ("gazutar", gazutar_config(s), decode_weight_bytes(s, batch, True), s["layers"])]
+
+    return _beside(args, batch, prompt_len, "sikevik", "Sanevik", models, ("sanevik", "zedirax", "gazutar"),
+                   ["sikevik", "sanevik", "zedirax", "gazutar"])

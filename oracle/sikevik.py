@@ -57,10 +57,11 @@ def begin_pass(x, e, w_loop):
 
 
 def visible(T, window, kept):
-    """[T, T] bool: key j is seen from position i"""
+    """[T, T] bool: key j is seen from position i (window None: every key up to i)"""
     i, j = torch.arange(T).view(T, 1), torch.arange(T).view(1, T)
-    inside = (j < kept) if window is None else (i - j < window) | (j < kept)
-    return (j <= i) & (inside if window is not None else torch.ones_like(inside))
+    if window is None:
+        return j <= i
+    return (j <= i) & ((i - j < window) | (j < kept))
 
 
 def softmax_with_one(s):
