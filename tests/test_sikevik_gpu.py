@@ -585,7 +585,7 @@ def test_passes_do_not_share_their_pages():
             r.close()
 
 
-def test_head_norm_weights_differ_by_channel_and_side(monkeypatch):
+def test_head_norm_weights_differ_by_channel_and_side():
     """Query and key norm weights that each silence half of the channels: swapped, missing or one-plus weights show."""
     cfg = config([with_mlp(attention(heads=4, kv_heads=2, dim=16, vdim=16, window=40, scale=1.0), None)], width=48, vocab=31)
     w = S.random_model(cfg, seed=16)
